@@ -5,5 +5,7 @@ from .botulorn import BotulornConfig
 from .fiterax import FiteraxConfig
 from .gilozen import GilozenConfig
 from .qwen2 import Qwen2Config
+from .romepel import RomepelConfig
 
-__all__ = ["BotulornConfig", "ConfigError", "FiteraxConfig", "GilozenConfig", "ModelConfig", "Qwen2Config", "read_config_json"]
+__all__ = ["BotulornConfig", "ConfigError", "FiteraxConfig", "GilozenConfig", "ModelConfig", "Qwen2Config",
+           "RomepelConfig", "read_config_json"]

@@ -41,13 +41,19 @@ class LatentAttentionConfig:
 class GLAConfig:
     """``heads`` heads of ``dim`` key channels and ``vdim`` value columns; decays sigmoid(z)^(1/tau), made through
     a bottleneck of ``decay_rank`` values.  config.json need not state that rank (key ``a_rank``): the shape of
-    the layer's ``mix.a1`` tensor gives it (``GilozenConfig.completed_from``)."""
+    the layer's ``mix.a1`` tensor gives it (``with_decay_ranks``)."""
 
     heads: int
     dim: int
     vdim: int
     tau: float
     decay_rank: Optional[int] = None
+
+    @classmethod
+    def from_mixer(cls, m: Mapping, where: str) -> "GLAConfig":
+        return cls(heads=_mixer_int(m, "heads", where), dim=_mixer_int(m, "dim", where), vdim=_mixer_int(m, "vdim", where),
+                   tau=checked_float(m.get("tau"), f"{where}.tau"),
+                   decay_rank=_mixer_int(m, "a_rank", where) if m.get("a_rank") is not None else None)
 
     def to_dict(self) -> dict:
         d = {"heads": self.heads, "dim": self.dim, "vdim": self.vdim, "tau": self.tau}
@@ -71,6 +77,20 @@ def _mixer_int(m: Mapping, key: str, where: str, minimum: int = 1) -> int:
     if key not in m:
         raise ConfigError(f"config.json: {where} has no '{key}'")
     return checked_int(m[key], f"{where}.{key}", minimum)
+
+
+def with_decay_ranks(layers, tensor_shapes: Mapping[str, tuple]) -> tuple:
+    """The layers (of any architecture) with the decay ranks that config.json left out filled in from the tensors."""
+    out = []
+    for i, layer in enumerate(layers):
+        name = f"l{i}.mix.a1"
+        if isinstance(layer.mixer, GLAConfig) and layer.mixer.decay_rank is None and name in tensor_shapes:
+            shape = tuple(tensor_shapes[name])
+            if len(shape) != 2 or shape[0] < 1:
+                raise ConfigError(f"tensor {name}: shape {shape} does not give the rank of the decays' bottleneck")
+            layer = replace(layer, mixer=replace(layer.mixer, decay_rank=int(shape[0])))
+        out.append(layer)
+    return tuple(out)
 
 
 @dataclass(frozen=True)
@@ -122,9 +142,7 @@ class GilozenConfig(ModelConfig):
                                                                                  mixer.rot_base, mixer.rot_dims):
                         raise ConfigError(f"config.json: {where} and layer {kv_from} must agree in kv_rank, rot_dim and rot")
             elif kind == GLA:
-                mixer = GLAConfig(heads=_mixer_int(m, "heads", where), dim=_mixer_int(m, "dim", where),
-                                  vdim=_mixer_int(m, "vdim", where), tau=checked_float(m.get("tau"), f"{where}.tau"),
-                                  decay_rank=_mixer_int(m, "a_rank", where) if m.get("a_rank") is not None else None)
+                mixer = GLAConfig.from_mixer(m, where)
             else:
                 raise ConfigError(f"config.json: {where}.type '{kind}' is not a mixer of this architecture "
                                   f"({LATENT}, {GLA})")
@@ -143,16 +161,7 @@ class GilozenConfig(ModelConfig):
                    layers=tuple(layers), eos_token_id=end_token_of(raw))
 
     def completed_from(self, tensor_shapes: Mapping[str, tuple]) -> "GilozenConfig":
-        layers = []
-        for i, layer in enumerate(self.layers):
-            name = f"l{i}.mix.a1"
-            if layer.kind == GLA and layer.mixer.decay_rank is None and name in tensor_shapes:
-                shape = tuple(tensor_shapes[name])
-                if len(shape) != 2 or shape[0] < 1:
-                    raise ConfigError(f"tensor {name}: shape {shape} does not give the rank of the decays' bottleneck")
-                layer = replace(layer, mixer=replace(layer.mixer, decay_rank=int(shape[0])))
-            layers.append(layer)
-        return replace(self, layers=tuple(layers))
+        return replace(self, layers=with_decay_ranks(self.layers, tensor_shapes))
 
     def to_dict(self) -> dict:
         d = {"architecture": self.architecture, "width": self.width, "vocab": self.vocab, "norm": {"eps": self.norm_eps},

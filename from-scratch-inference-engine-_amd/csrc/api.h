@@ -45,9 +45,11 @@ int fsie_device_info(char* arch_out, int arch_len, int* n_compute_units);
 // Compute units of the current device; 0 if there is no device to ask.
 int fsie_device_compute_units(void);
 
-// out[t] = table[ids[t]] * scale, float32
+// out[t] = table[ids[t]] * scale + pos_table[positions[t]], float32; pos_table (n_positions rows of the table's type,
+// with positions) or null for no second term.  A row that does not exist counts as zeros.
 int fsie_embedding(const void* table, int dtype, const int32_t* ids, float* out, int n_tokens, int hidden,
-                   int vocab, float scale, hipStream_t stream);
+                   int vocab, float scale, const void* pos_table, const int32_t* positions, int n_positions,
+                   hipStream_t stream);
 int fsie_rmsnorm(float* residual, const void* delta, const float* weight, void* out, const int32_t* rows,
                  int n_rows, int hidden, float eps, int dtype, int write_back, int n_parts, int total_rows,
                  hipStream_t stream);
@@ -67,10 +69,11 @@ int fsie_swiglu(const void* x, void* out, int n_tokens, int inter, int dtype, hi
 int fsie_gated_act(const void* x, void* out, int n_tokens, int inter, int dtype, int act, hipStream_t stream);
 // The norm of a sublayer's output, the residual sum and the next norm in one pass:
 //   v = residual + rmsnorm(delta; post_weight, post_eps);  out = rmsnorm(v; weight, eps)
-// delta as for fsie_rmsnorm (one array of the activations' type, or n_parts float32 partial sums).
-int fsie_sandwich_norm(float* residual, const void* delta, const float* post_weight, float post_eps, const float* weight,
-                       float eps, void* out, const int32_t* rows, int n_rows, int hidden, int dtype, int write_back,
-                       int n_parts, int total_rows, hipStream_t stream);
+// delta as for fsie_rmsnorm (one array of the activations' type, or n_parts float32 partial sums), plus delta_bias
+// [hidden] in every row (or null).
+int fsie_sandwich_norm(float* residual, const void* delta, const float* delta_bias, const float* post_weight,
+                       float post_eps, const float* weight, float eps, void* out, const int32_t* rows, int n_rows,
+                       int hidden, int dtype, int write_back, int n_parts, int total_rows, hipStream_t stream);
 // out[t][h][:] = rmsnorm(o[t][h][:]; weight, eps) * act(gate[t][h][:]), a head `width` values wide; o float32, the sum
 // in order of n_planes arrays [n_tokens][heads * width] that lie one after the other
 int fsie_gated_headnorm(const float* o, int n_planes, const void* gate, int64_t gate_stride, const float* weight, void* out,
@@ -113,7 +116,14 @@ int fsie_residual_add(float* residual, const void* delta, int64_t total, int dty
 int fsie_bias_add(void* y, const float* bias, int rows, int cols, int dtype, hipStream_t stream);
 // y [rows][cols] bfloat16 = parts[0] + parts[1] + ... (float32 [planes][rows][cols], added in their order) + bias
 // (float32 [cols] or null), rounded once; cols a multiple of 4
-int fsie_sum_round(const float* parts, int planes, const float* bias, void* y, int rows, int cols, hipStream_t stream);
+// (act, act_pos, act_neg: an activation of the sum before it is rounded, FsiePointAct; 0: none)
+int fsie_sum_round(const float* parts, int planes, const float* bias, void* y, int rows, int cols, int act, float act_pos,
+                   float act_neg, hipStream_t stream);
+// y = act(x + bias) over rows of `cols` values (bias float32 [cols] or null; y may be x; act: FsiePointAct)
+int fsie_bias_act(const void* x, const float* bias, void* y, int rows, int cols, int dtype, int act, float act_pos,
+                  float act_neg, hipStream_t stream);
+// out[t] = 1 + coef * ln(floor((positions[t] + 1) / every) + 1)
+int fsie_query_temperature(const int32_t* positions, int n_tokens, double coef, double every, float* out, hipStream_t stream);
 
 int fsie_rope_kv_write(void* qkv, const int32_t* positions, const int32_t* slots, const double* inv_freq,
                        const float* bias, void* k_pool, void* v_pool, int n_tokens, int n_heads, int n_kv, int head_dim,
@@ -191,6 +201,13 @@ int fsie_gemm_mfma_wide_gated(const void* x, const void* w, void* y, int M, int 
 // whether they take M rows of this shape (65 to FSIE_GEMM_MFMA_WIDE_MAX_M rows: only some launch shapes on a
 // fragment-ordered weight)
 int fsie_gemm_mfma_wide_takes(int M, int N, int K, int splits, int gate_up, int frags);
+// y = act(x . w^T + bias) in bfloat16, act a FsiePointAct with its constants: by the few-rows product (up to 16 rows) and
+// by the one that shares x through LDS (its rows; one slice of K, N a multiple of 4)
+int fsie_gemm_mfma_skinny_act(const void* x, const void* w, const float* bias, void* y, int M, int N, int K, int waves,
+                              int blocks, int act, float act_pos, float act_neg, hipStream_t stream);
+int fsie_gemm_mfma_wide_act(const void* x, const void* w, const float* bias, void* y, int M, int N, int K, int waves,
+                            int blocks, int frags, int act, float act_pos, float act_neg, hipStream_t stream);
+int fsie_gemm_mfma_wide_act_takes(int M, int N, int K, int frags);
 int64_t fsie_fragment_order_size(int N, int K);
 int fsie_fragment_order(const void* w, void* out, int N, int K, hipStream_t stream);
 
@@ -199,13 +216,17 @@ int fsie_attention_scalar(const void* q, int64_t q_stride, const void* k_pool, c
                           void* out, float* partials, int n_heads, int n_kv, int head_dim, int page_size,
                           int window, float scale, int dtype, const float* sinks, float softcap, const void* k_pooled,
                           const void* v_pooled, const int32_t* pooled_tables, int pooled_max_pages, int pooled_page_size,
-                          int pooled_tokens, hipStream_t stream);
+                          int pooled_tokens, const float* slopes, const float* row_scale, hipStream_t stream);
 // k_pooled .. pooled_tokens (or null and zeros): pools [units][n_kv][pooled_page_size][head_dim] and
 // [units][n_kv][head_dim][pooled_page_size] that hold one mean key and value for every block of pooled_tokens positions,
 // with their block table [requests][pooled_max_pages]; an item flagged FSIE_ATTN_POOL_WALK reads, beside its own keys,
 // the blocks that lie wholly before a query's window (fsie_pool_blocks fills them).
 // softcap (in every attention entry point that takes it): a positive number caps the scaled scores,
 // s <- softcap * tanh(s / softcap), before the mask and the softmax; 0: scores as they are.
+// slopes (or null, in every attention entry point that takes it): float32 [n_heads]; slopes[h] * (query position - key
+// position) is taken off the scores of head h, behind the scale and the cap.
+// row_scale (or null, in every attention entry point that takes it): float32, a factor for every row of q on all its
+// scores, before the cap.
 // sinks (or null, in every attention entry point that takes it): float32 [n_heads]; exp(sinks[h]) is one more
 // term of the softmax denominator of every query row of head h.  It has no key and no value and is not scaled.
 // Items that leave partial records ignore it; the merge that combines them adds it once.
@@ -224,20 +245,22 @@ int fsie_pool_blocks(const void* k_pool, const void* v_pool, const int32_t* bloc
 int fsie_attention_mfma(const void* q, int64_t q_stride, const void* k_pool, const void* v_pool,
                         const int32_t* block_tables, int max_pages, const int32_t* items, int n_items, void* out,
                         float* partials, int n_heads, int n_kv, int head_dim, int page_size, int window, float scale,
-                        int large, int waves, const float* sinks, float softcap, hipStream_t stream);
+                        int large, int waves, const float* sinks, float softcap, const float* slopes,
+                        const float* row_scale, hipStream_t stream);
 // the same for a step of one token a request, from the q/k/v product's partial sums: bias, rotation and the
-// write into the pools happen in the kernel
+// write into the pools happen in the kernel (cos_sin null: no rotation)
 int fsie_attention_mfma_qkv_ok(int head_dim, int page_size);
 int fsie_attention_mfma_qkv(const float* sums, int n_parts, int n_tokens, const float* bias, const float* cos_sin,
                             const int32_t* slots, void* k_pool, void* v_pool, int64_t pool_slots,
                             const int32_t* block_tables, int max_pages, const int32_t* items, int n_items, void* out,
                             float* partials, int n_heads, int n_kv, int head_dim, int page_size, int window,
-                            float scale, int waves, hipStream_t stream);
+                            float scale, int waves, const float* slopes, const float* row_scale, hipStream_t stream);
 int fsie_attention_mfma_lds_ok(int head_dim, int page_size);
 int fsie_attention_mfma_lds(const void* q, int64_t q_stride, const void* k_pool, const void* v_pool,
                             const int32_t* block_tables, int max_pages, const int32_t* items, const int32_t* groups,
                             int n_groups, void* out, int n_heads, int n_kv, int head_dim, int page_size, int window,
-                            float scale, const float* sinks, float softcap, hipStream_t stream);
+                            float scale, const float* sinks, float softcap, const float* slopes, const float* row_scale,
+                            hipStream_t stream);
 int fsie_attention_mfma_tiles(int head_dim, int large);
 int fsie_attention_mfma_max_waves(int head_dim);
 

@@ -72,7 +72,7 @@ __device__ __forceinline__ uint2 ld8(const bf16_t* p) { return *reinterpret_cast
 struct QkvSums {
     const float* sums;     // [n_parts][n_tokens][width], width = (n_heads + 2 n_kv) head_dim
     const float* bias;     // [width], or null
-    const float* cos_sin;  // [n_tokens][head_dim / 2] pairs (cos, sin) of each token's position
+    const float* cos_sin;  // [n_tokens][head_dim / 2] pairs (cos, sin) of each token's position, or null: no rotation
     const int32_t* slots;  // [n_tokens] slot of a token's key and value in the pools (negative: nowhere)
     bf16_t* k_out;         // the pools again, to write
     bf16_t* v_out;
@@ -81,6 +81,9 @@ struct QkvSums {
     int n_parts, width;
     const float* sinks;    // [n_heads] or null: exp(sink) joins every row's denominator (any variant)
     float softcap;         // > 0: the scaled scores become softcap * tanh(score / softcap) (any variant); 0: as they are
+    const float* slopes;     // [n_heads] or null: slopes[h] * (query position - key position) is taken off the (capped)
+                             // scores of head h (any variant)
+    const float* row_scale;  // [n_tokens] or null: a factor on all scores of a token, before the cap (any variant)
 };
 
 // Element d of a head after the rotation of the pairs (i, i + HD / 2) by the angles whose
@@ -174,8 +177,10 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
     const float scale2 = scale * kLog2e;  // scores in units of log2 e: exp() becomes exp2()
     // capped scores: softcap * tanh(product * scale / softcap), in the same units
     const bool capped = f.softcap > 0.f;
-    const float cap2 = f.softcap * kLog2e, cap_in = capped ? scale / f.softcap : 0.f;
-    auto scaled = [&](float product) { return capped ? cap2 * tanh_by_exp(product * cap_in) : product * scale2; };
+    const float cap2 = f.softcap * kLog2e, cap_in = capped ? scale / f.softcap : scale2;
+    auto scaled = [&](float product, float in) { return capped ? cap2 * tanh_by_exp(product * in) : product * in; };
+    // the distance bias, in the same units: slope (key - query), added to the scaled scores
+    const bool sloped = f.slopes != nullptr;
 
     // LDS: the accumulators that the waves after the first hand over at the end; before that, in
     // the QKV variant, the heads added up from the sums (up to 16 of queries, a key, a value) and
@@ -231,8 +236,10 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
                 part[j][u] = *reinterpret_cast<const float4*>(col_at[j] + min(u, f.n_parts - 1) * f.part_stride);
             bias_of[j] = *reinterpret_cast<const float4*>(f.bias ? f.bias + col : col_at[j]);
         }
-        const float2* cs = reinterpret_cast<const float2*>(f.cos_sin) + static_cast<int64_t>(q_row0) * (HD / 2);
-        angle = cs[min(max(sum_thread, 0), HD / 2 - 1)];
+        if (f.cos_sin) {
+            const float2* cs = reinterpret_cast<const float2*>(f.cos_sin) + static_cast<int64_t>(q_row0) * (HD / 2);
+            angle = cs[min(max(sum_thread, 0), HD / 2 - 1)];
+        }
     };
     auto finish_sums = [&]() {
 #pragma unroll
@@ -251,7 +258,7 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
             if (lds_at[j] >= 0) *reinterpret_cast<float4*>(s_row + lds_at[j]) = a;
         }
         for (int i = max(sum_thread, 0); i < HD / 2; i += sum_threads) {
-            if (i == sum_thread) s_cs[i] = angle;
+            if (i == sum_thread || !f.cos_sin) s_cs[i] = angle;  // (without a table: cosine 1, sine 0)
             else s_cs[i] = (reinterpret_cast<const float2*>(f.cos_sin) + static_cast<int64_t>(q_row0) * (HD / 2))[i];
         }
     };
@@ -259,6 +266,7 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
     // ---- the item's queries: B operands, kept for the whole item
     bool rvalid[NT];
     int rpos[NT], rtok[NT], rhead[NT];
+    float r_in[NT], r_slope[NT];  // the row's factor from products to scores, and its head's slope
     F16B qf[NT][S32A];
     F8B qt[NT][S16A];
 #pragma unroll
@@ -269,6 +277,8 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
         rtok[nt] = tq;
         rhead[nt] = h_base + hh;
         rpos[nt] = pos0 + tq;
+        r_in[nt] = f.row_scale ? cap_in * f.row_scale[q_row0 + (rvalid[nt] ? tq : 0)] : cap_in;
+        r_slope[nt] = sloped ? f.slopes[rvalid[nt] ? rhead[nt] : h_base] * kLog2e : 0.f;
         if constexpr (!QKV) {
             const bf16_t* qp = q + static_cast<int64_t>(q_row0 + (rvalid[nt] ? tq : 0)) * q_stride +
                                static_cast<int64_t>(rvalid[nt] ? rhead[nt] : h_base) * HD;
@@ -421,10 +431,7 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
             float m_loc = -INFINITY;
             if (full) {
 #pragma unroll
-                for (int i = 0; i < 8; ++i) {
-                    sv[i] = scaled(st[i >> 2][i & 3]);
-                    m_loc = fmaxf(m_loc, sv[i]);
-                }
+                for (int i = 0; i < 8; ++i) sv[i] = scaled(st[i >> 2][i & 3], r_in[nt]);
             } else {
 #pragma unroll
                 for (int t = 0; t < 2; ++t)
@@ -434,10 +441,16 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
                         const bool in_range = kept_block ? key < prefix_end : (key >= key_begin && key < key_end);
                         const bool vis = rvalid[nt] && in_range && key <= rpos[nt] &&
                                          (window <= 0 || key > rpos[nt] - window || key < keep);
-                        sv[t * 4 + r] = vis ? scaled(st[t][r]) : -INFINITY;
-                        m_loc = fmaxf(m_loc, sv[t * 4 + r]);
+                        sv[t * 4 + r] = vis ? scaled(st[t][r], r_in[nt]) : -INFINITY;
                     }
             }
+            if (sloped) {  // (the same for the whole launch; hidden keys stay at minus infinity)
+                const float at_first = r_slope[nt] * static_cast<float>(kb + 8 * G - rpos[nt]);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) sv[i] += fmaf(r_slope[nt], static_cast<float>(i), at_first);
+            }
+#pragma unroll
+            for (int i = 0; i < 8; ++i) m_loc = fmaxf(m_loc, sv[i]);
             m_loc = max_xor32(max_xor16(m_loc));
             const float m_new = fmaxf(m_run[nt], m_loc);
             const float corr = (m_run[nt] == -INFINITY) ? 1.f : __builtin_amdgcn_exp2f(m_run[nt] - m_new);
@@ -710,11 +723,14 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
 template <int HDT, int NT>
 int launch(const void* q, int64_t q_stride, const void* k_pool, const void* v_pool, const int32_t* block_tables,
            int max_pages, const int32_t* items, int n_items, void* out, float* partials, int n_heads, int n_kv,
-           int page_size, int window, float scale, int waves, const float* sinks, float softcap, hipStream_t stream) {
+           int page_size, int window, float scale, int waves, const float* sinks, float softcap, const float* slopes,
+           const float* row_scale, hipStream_t stream) {
     constexpr int MAXW = NT == 1 ? max_waves<HDT>() : 4;
-    QkvSums only_sinks{};
-    only_sinks.sinks = sinks;
-    only_sinks.softcap = softcap;
+    QkvSums scores{};
+    scores.sinks = sinks;
+    scores.softcap = softcap;
+    scores.slopes = slopes;
+    scores.row_scale = row_scale;
     const int group = n_heads / n_kv;
     const int rows = 16 * NT;
     const int gh = group < rows ? group : rows;
@@ -728,7 +744,7 @@ int launch(const void* q, int64_t q_stride, const void* k_pool, const void* v_po
     attention_mfma_kernel<HDT, NT, W, V><<<grid, THREADS, 0, stream>>>(                                              \
         static_cast<const bf16_t*>(q), q_stride, static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool), \
         block_tables, max_pages, items, static_cast<bf16_t*>(out), partials, n_heads, n_kv, page_size, window, scale, \
-        gh, head_chunks, only_sinks)
+        gh, head_chunks, scores)
     const bool v16 = page_size % 8 == 0;
     if (waves == 1) {
         if (v16) FSIE_ATTN_LAUNCH(1, 64, true);
@@ -771,6 +787,6 @@ typedef int (*LaunchQkvFn)(const QkvSums&, const void*, const void*, const int32
                            float*, int, int, int, int, float, int, hipStream_t);
 
 typedef int (*LaunchFn)(const void*, int64_t, const void*, const void*, const int32_t*, int, const int32_t*, int, void*,
-                        float*, int, int, int, int, float, int, const float*, float, hipStream_t);
+                        float*, int, int, int, int, float, int, const float*, float, const float*, const float*, hipStream_t);
 
 }  // namespace fsie_attn

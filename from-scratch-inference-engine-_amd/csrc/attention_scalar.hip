@@ -55,7 +55,8 @@ __global__ __launch_bounds__(256) void attention_scalar_kernel(
     T* __restrict__ out, float* __restrict__ partials, int n_heads, int n_kv, int hd, int page_size,
     int window, float scale, int gh, int head_chunks, const float* __restrict__ sinks, float softcap,
     const T* __restrict__ k_pooled, const T* __restrict__ v_pooled, const int32_t* __restrict__ pooled_tables,
-    int pooled_max_pages, int pooled_page_size, int pooled_tokens) {
+    int pooled_max_pages, int pooled_page_size, int pooled_tokens, const float* __restrict__ slopes,
+    const float* __restrict__ row_scale) {
     extern __shared__ float lds[];
     float* qs = lds;                          // [kRows][hd]
     float* kv = qs + kRows * hd;              // [kKeys][hd + 1]
@@ -105,9 +106,15 @@ __global__ __launch_bounds__(256) void attention_scalar_kernel(
         qs[e] = v;
     }
 
+    // the factor of a row's token on its scores and the slope of its head's distance bias
+    float r_scale[2], r_slope[2];
     float m_run[2], l_run[2], acc[2][MAXC];
 #pragma unroll
     for (int p = 0; p < 2; ++p) {
+        const int r = wave * 4 + p * 2 + sub;
+        const bool row_ok = r < n_rows && (r % gh) < gh_here;
+        r_scale[p] = row_ok && row_scale ? scale * row_scale[q_row0 + r / gh] : scale;
+        r_slope[p] = row_ok && slopes ? slopes[h_base + (r % gh)] : 0.f;
         m_run[p] = -INFINITY;
         l_run[p] = 0.f;
 #pragma unroll
@@ -175,8 +182,9 @@ __global__ __launch_bounds__(256) void attention_scalar_kernel(
                 const float* kr = kv + lane32 * kv_stride;
                 float dot = 0.f;
                 for (int d = 0; d < hd; ++d) dot = fmaf(qr[d], kr[d], dot);
-                s = dot * scale;
+                s = dot * r_scale[p];
                 if (softcap > 0.f) s = softcap * tanhf(s / softcap);  // capped scores: softcap * tanh(s / softcap)
+                if (slopes) s = fmaf(r_slope[p], static_cast<float>(kj - pos), s);
             }
             const float m_new = fmaxf(m_run[p], half_wave_max(s));
             const float pe = (s == -INFINITY) ? 0.f : expf(s - m_new);
@@ -459,7 +467,8 @@ extern "C" int fsie_attention_scalar(const void* q, int64_t q_stride, const void
                                      int head_dim, int page_size, int window, float scale, int dtype,
                                      const float* sinks, float softcap, const void* k_pooled, const void* v_pooled,
                                      const int32_t* pooled_tables, int pooled_max_pages, int pooled_page_size,
-                                     int pooled_tokens, hipStream_t stream) {
+                                     int pooled_tokens, const float* slopes, const float* row_scale, hipStream_t stream) {
+    FSIE_REQUIRE(!(k_pooled && slopes), "attention: a distance bias over pooled blocks has no meaning (a block has no one position)");
     FSIE_REQUIRE(!k_pooled || (v_pooled && pooled_tables && pooled_max_pages > 0 && pooled_page_size > 0 && pooled_tokens > 0 &&
                                window > 0),
                  "attention: pooled blocks come with their pools, tables, a block size and a window");
@@ -493,7 +502,7 @@ extern "C" int fsie_attention_scalar(const void* q, int64_t q_stride, const void
                                            static_cast<T*>(out), partials, n_heads, n_kv, head_dim, page_size, window, \
                                            scale, gh, head_chunks, sinks, softcap, static_cast<const T*>(k_pooled),  \
                                            static_cast<const T*>(v_pooled), pooled_tables, pooled_max_pages,         \
-                                           pooled_page_size, pooled_tokens);                                         \
+                                           pooled_page_size, pooled_tokens, slopes, row_scale);                      \
     } while (0)
 #define FSIE_SCALAR_ATTENTION_OF(T)                                          \
     if (wide) {                                                              \

@@ -64,6 +64,16 @@ __device__ __forceinline__ float gate_act(float g, int act) {
     return g / (1.0f + expf(-g));
 }
 
+// ---- activations of one value (a feed-forward without a gate) ------------------------------
+// 1: xIELU, z / 2 plus pos * z^2 above zero and neg * (exp(z) - 1 - z) below it.
+enum FsiePointAct { FSIE_POINT_NONE = 0, FSIE_POINT_XIELU = 1 };
+#define FSIE_POINT_KNOWN(act) ((act) == FSIE_POINT_NONE || (act) == FSIE_POINT_XIELU)
+__device__ __forceinline__ float point_act(float z, int act, float pos, float neg) {
+    if (act == FSIE_POINT_NONE) return z;
+    const float below = fminf(z, 0.f);
+    return fmaf(0.5f, z, z > 0.f ? pos * z * z : neg * (expm1f(below) - below));
+}
+
 // tanh through one exponential, 1 - 2 / (exp(2x) + 1): within a few float32 roundings of 1 in absolute terms,
 // right at both ends (exp overflows to infinity: 1; underflows to 0: -1); for score caps in kernels that
 // work in bfloat16 anyway.  Float32 paths call tanhf.

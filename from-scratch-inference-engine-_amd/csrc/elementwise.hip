@@ -9,20 +9,22 @@ namespace {
 constexpr int kThreads = 256;
 constexpr int kWideNormRows = 128;  // up to so many rows (half the device's units), RMSNorm runs in workgroups of 1,024 threads
 
-// out[t, :] = table[ids[t], :] as float32.  An id outside the table gives a row of zeros; the
-// host refuses such ids before the launch.
+// out[t, :] = table[ids[t], :] * scale as float32, plus the position's row of a second table if there is one.  An id or a
+// position outside its table counts as a row of zeros; the host refuses such ids and positions before the launch.
 template <typename T>
 __global__ void embedding_kernel(const T* __restrict__ table, const int32_t* __restrict__ ids,
-                                 float* __restrict__ out, int hidden, int vocab, float scale) {
+                                 float* __restrict__ out, int hidden, int vocab, float scale,
+                                 const T* __restrict__ pos_table, const int32_t* __restrict__ positions, int n_positions) {
     const int t = blockIdx.x;
     const int id = ids[t];
+    const int pos = pos_table ? positions[t] : -1;
     float* dst = out + static_cast<int64_t>(t) * hidden;
-    if (id < 0 || id >= vocab) {
-        for (int j = threadIdx.x; j < hidden; j += blockDim.x) dst[j] = 0.f;
-        return;
+    const T* src = id >= 0 && id < vocab ? table + static_cast<int64_t>(id) * hidden : nullptr;
+    const T* place = pos >= 0 && pos < n_positions ? pos_table + static_cast<int64_t>(pos) * hidden : nullptr;
+    for (int j = threadIdx.x; j < hidden; j += blockDim.x) {
+        const float v = src ? to_float(src[j]) * scale : 0.f;
+        dst[j] = place ? v + to_float(place[j]) : v;
     }
-    const T* src = table + static_cast<int64_t>(id) * hidden;
-    for (int j = threadIdx.x; j < hidden; j += blockDim.x) dst[j] = to_float(src[j]) * scale;
 }
 
 // One block per output row r; source row = rows ? rows[r] : r.
@@ -93,7 +95,9 @@ struct Pack4<bf16_t> {
 // four elements per thread, grid = (tokens, quads / threads): no loop, one load per thread
 template <typename T>
 __global__ void embedding_vec_kernel(const T* __restrict__ table, const int32_t* __restrict__ ids,
-                                     float* __restrict__ out, int hidden, int vocab, float scale) {
+                                     float* __restrict__ out, int hidden, int vocab, float scale,
+                                     const T* __restrict__ pos_table, const int32_t* __restrict__ positions,
+                                     int n_positions) {
     const int t = blockIdx.x;
     const int j = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
     if (j >= hidden) return;
@@ -101,7 +105,15 @@ __global__ void embedding_vec_kernel(const T* __restrict__ table, const int32_t*
     const bool ok = id >= 0 && id < vocab;
     float4 v = Pack4<T>::load(table + static_cast<int64_t>(ok ? id : 0) * hidden + j);
     v = float4{v.x * scale, v.y * scale, v.z * scale, v.w * scale};  // (times 1 changes no bit)
-    Pack4<float>::store(out + static_cast<int64_t>(t) * hidden + j, ok ? v : float4{0.f, 0.f, 0.f, 0.f});
+    if (!ok) v = float4{0.f, 0.f, 0.f, 0.f};
+    if (pos_table) {
+        const int pos = positions[t];
+        if (pos >= 0 && pos < n_positions) {
+            const float4 p = Pack4<T>::load(pos_table + static_cast<int64_t>(pos) * hidden + j);
+            v = float4{v.x + p.x, v.y + p.y, v.z + p.z, v.w + p.w};
+        }
+    }
+    Pack4<float>::store(out + static_cast<int64_t>(t) * hidden + j, v);
 }
 
 // DELTA: 0 = none, 1 = one array of T, 2 to 9 = that many float32 partial sums, added in
@@ -306,9 +318,37 @@ __global__ void bias_add_kernel(T* __restrict__ y, const float* __restrict__ bia
     if (i < total) y[i] = from_float<T>(to_float(y[i]) + bias[i % cols]);
 }
 
-// y = sum of `planes` float32 partial sums, added in their order, + bias, rounded once; four values a thread
+// y = act(x + bias), one row a blockIdx.x; VEC: four values a thread
+template <typename T, bool VEC>
+__global__ __launch_bounds__(kThreads) void bias_act_kernel(const T* __restrict__ x, const float* __restrict__ bias, T* __restrict__ y,
+                                                            int cols, int act, float act_pos, float act_neg) {
+    const int j = (blockIdx.y * kThreads + threadIdx.x) * (VEC ? 4 : 1);
+    if (j >= cols) return;
+    const int64_t i = static_cast<int64_t>(blockIdx.x) * cols + j;
+    if constexpr (VEC) {
+        float4 v = Pack4<T>::load(x + i);
+        if (bias) {
+            const float4 b = Pack4<float>::load(bias + j);
+            v = float4{v.x + b.x, v.y + b.y, v.z + b.z, v.w + b.w};
+        }
+        Pack4<T>::store(y + i, float4{point_act(v.x, act, act_pos, act_neg), point_act(v.y, act, act_pos, act_neg),
+                                      point_act(v.z, act, act_pos, act_neg), point_act(v.w, act, act_pos, act_neg)});
+    } else {
+        y[i] = from_float<T>(point_act(to_float(x[i]) + (bias ? bias[j] : 0.f), act, act_pos, act_neg));
+    }
+}
+
+// The factor on a token's scores that grows with the logarithm of its position's period; float64 inside, so that
+// the quotient's floor is exact at the periods' ends.
+__global__ void query_temperature_kernel(const int32_t* __restrict__ positions, int n_tokens, double coef, double every,
+                                         float* __restrict__ out) {
+    const int t = blockIdx.x * blockDim.x + threadIdx.x;
+    if (t < n_tokens) out[t] = static_cast<float>(1.0 + coef * log(floor((positions[t] + 1.0) / every) + 1.0));
+}
+
+// y = act(sum of `planes` float32 partial sums, added in their order, + bias), rounded once; four values a thread
 __global__ void sum_round_kernel(const float* __restrict__ parts, int planes, int64_t plane, const float* __restrict__ bias,
-                                 bf16_t* __restrict__ y, int64_t total, int cols) {
+                                 bf16_t* __restrict__ y, int64_t total, int cols, int act, float act_pos, float act_neg) {
     const int64_t i = (static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x) * 4;
     if (i >= total) return;
     float4 sum = *reinterpret_cast<const float4*>(parts + i);
@@ -320,6 +360,9 @@ __global__ void sum_round_kernel(const float* __restrict__ parts, int planes, in
         const float4 b = *reinterpret_cast<const float4*>(bias + i % cols);
         sum.x += b.x, sum.y += b.y, sum.z += b.z, sum.w += b.w;
     }
+    if (act != FSIE_POINT_NONE)
+        sum = float4{point_act(sum.x, act, act_pos, act_neg), point_act(sum.y, act, act_pos, act_neg),
+                     point_act(sum.z, act, act_pos, act_neg), point_act(sum.w, act, act_pos, act_neg)};
     uint2 raw;
     raw.x = static_cast<uint32_t>(from_float<bf16_t>(sum.x).bits) | static_cast<uint32_t>(from_float<bf16_t>(sum.y).bits) << 16;
     raw.y = static_cast<uint32_t>(from_float<bf16_t>(sum.z).bits) | static_cast<uint32_t>(from_float<bf16_t>(sum.w).bits) << 16;
@@ -485,19 +528,21 @@ extern "C" int fsie_rmsnorm_plain(const void* x, int64_t x_stride, const float* 
 }
 
 extern "C" int fsie_embedding(const void* table, int dtype, const int32_t* ids, float* out,
-                              int n_tokens, int hidden, int vocab, float scale, hipStream_t stream) {
+                              int n_tokens, int hidden, int vocab, float scale, const void* pos_table,
+                              const int32_t* positions, int n_positions, hipStream_t stream) {
     FSIE_REQUIRE(n_tokens >= 0 && hidden > 0 && vocab > 0, "embedding: bad sizes T=%d H=%d V=%d",
                  n_tokens, hidden, vocab);
     FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "embedding: unknown dtype %d", dtype);
+    FSIE_REQUIRE(!pos_table || (positions && n_positions > 0), "embedding: a table of positions comes with positions and its size");
     if (n_tokens == 0) return 0;
-    const bool vec = hidden % 4 == 0 && reinterpret_cast<uintptr_t>(table) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
+    const bool vec = hidden % 4 == 0 && reinterpret_cast<uintptr_t>(table) % 16 == 0 && reinterpret_cast<uintptr_t>(pos_table) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
     const dim3 vgrid(n_tokens, static_cast<unsigned>(ceil_div64(hidden / 4, kThreads)));
     if (dtype == FSIE_F32) {
-        if (vec) embedding_vec_kernel<float><<<vgrid, kThreads, 0, stream>>>(static_cast<const float*>(table), ids, out, hidden, vocab, scale);
-        else embedding_kernel<float><<<n_tokens, kThreads, 0, stream>>>(static_cast<const float*>(table), ids, out, hidden, vocab, scale);
+        if (vec) embedding_vec_kernel<float><<<vgrid, kThreads, 0, stream>>>(static_cast<const float*>(table), ids, out, hidden, vocab, scale, static_cast<const float*>(pos_table), positions, n_positions);
+        else embedding_kernel<float><<<n_tokens, kThreads, 0, stream>>>(static_cast<const float*>(table), ids, out, hidden, vocab, scale, static_cast<const float*>(pos_table), positions, n_positions);
     } else {
-        if (vec) embedding_vec_kernel<bf16_t><<<vgrid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(table), ids, out, hidden, vocab, scale);
-        else embedding_kernel<bf16_t><<<n_tokens, kThreads, 0, stream>>>(static_cast<const bf16_t*>(table), ids, out, hidden, vocab, scale);
+        if (vec) embedding_vec_kernel<bf16_t><<<vgrid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(table), ids, out, hidden, vocab, scale, static_cast<const bf16_t*>(pos_table), positions, n_positions);
+        else embedding_kernel<bf16_t><<<n_tokens, kThreads, 0, stream>>>(static_cast<const bf16_t*>(table), ids, out, hidden, vocab, scale, static_cast<const bf16_t*>(pos_table), positions, n_positions);
     }
     FSIE_CHECK_LAUNCH("embedding");
     return 0;
@@ -592,8 +637,9 @@ extern "C" int fsie_residual_add(float* residual, const void* delta, int64_t tot
     return 0;
 }
 
-extern "C" int fsie_sum_round(const float* parts, int planes, const float* bias, void* y, int rows, int cols,
-                              hipStream_t stream) {
+extern "C" int fsie_sum_round(const float* parts, int planes, const float* bias, void* y, int rows, int cols, int act,
+                              float act_pos, float act_neg, hipStream_t stream) {
+    FSIE_REQUIRE(FSIE_POINT_KNOWN(act), "sum_round: unknown activation %d", act);
     FSIE_REQUIRE(rows >= 0 && cols > 0 && cols % 4 == 0 && planes >= 1, "sum_round: bad sizes %d x %d, %d planes", rows, cols, planes);
     FSIE_REQUIRE(parts && y, "sum_round: missing operand");
     FSIE_REQUIRE((reinterpret_cast<uintptr_t>(parts) & 15) == 0 && (reinterpret_cast<uintptr_t>(bias) & 15) == 0 &&
@@ -601,8 +647,38 @@ extern "C" int fsie_sum_round(const float* parts, int planes, const float* bias,
     const int64_t total = static_cast<int64_t>(rows) * cols;
     if (total == 0) return 0;
     sum_round_kernel<<<static_cast<unsigned>(ceil_div64(total / 4, kThreads)), kThreads, 0, stream>>>(
-        parts, planes, total, bias, static_cast<bf16_t*>(y), total, cols);
+        parts, planes, total, bias, static_cast<bf16_t*>(y), total, cols, act, act_pos, act_neg);
     FSIE_CHECK_LAUNCH("sum_round");
+    return 0;
+}
+
+extern "C" int fsie_bias_act(const void* x, const float* bias, void* y, int rows, int cols, int dtype, int act,
+                             float act_pos, float act_neg, hipStream_t stream) {
+    FSIE_REQUIRE(rows >= 0 && cols > 0 && x && y, "bias_act: bad operands, %d x %d", rows, cols);
+    FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "bias_act: unknown dtype %d", dtype);
+    FSIE_REQUIRE(FSIE_POINT_KNOWN(act), "bias_act: unknown activation %d", act);
+    if (rows == 0) return 0;
+    const bool vec = cols % 4 == 0 && ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(y) |
+                                        reinterpret_cast<uintptr_t>(bias)) & 15) == 0;
+    const dim3 grid(static_cast<unsigned>(rows), static_cast<unsigned>(ceil_div64(vec ? cols / 4 : cols, kThreads)));
+#define FSIE_BIAS_ACT(T, V) \
+    bias_act_kernel<T, V><<<grid, kThreads, 0, stream>>>(static_cast<const T*>(x), bias, static_cast<T*>(y), cols, act, act_pos, act_neg)
+    if (dtype == FSIE_F32) {
+        if (vec) FSIE_BIAS_ACT(float, true); else FSIE_BIAS_ACT(float, false);
+    } else {
+        if (vec) FSIE_BIAS_ACT(bf16_t, true); else FSIE_BIAS_ACT(bf16_t, false);
+    }
+#undef FSIE_BIAS_ACT
+    FSIE_CHECK_LAUNCH("bias_act");
+    return 0;
+}
+
+extern "C" int fsie_query_temperature(const int32_t* positions, int n_tokens, double coef, double every, float* out,
+                                      hipStream_t stream) {
+    FSIE_REQUIRE(n_tokens >= 0 && positions && out && every > 0.0, "query_temperature: bad operands T=%d every=%f", n_tokens, every);
+    if (n_tokens == 0) return 0;
+    query_temperature_kernel<<<static_cast<unsigned>(ceil_div64(n_tokens, 64)), 64, 0, stream>>>(positions, n_tokens, coef, every, out);
+    FSIE_CHECK_LAUNCH("query_temperature");
     return 0;
 }
 

@@ -9,9 +9,11 @@
 // splits > 1: K is cut into that many slices, each summed by workgroups of its own; y is then
 // float32 [splits, M, N], partial sums without bias, which the consumer adds in the order of the slices
 // (fsie_rmsnorm takes them as its delta).  Every slice must hold at least 64 values of K.
-extern "C" int fsie_gemm_mfma_skinny(const void* x, const void* w, const float* bias, void* y, int M, int N, int K,
-                                     int out_f32, int waves, int blocks, int epilogue, int splits,
-                                     hipStream_t stream) {
+static int gemm_mfma_skinny(const void* x, const void* w, const float* bias, void* y, int M, int N, int K, int out_f32,
+                            int waves, int blocks, int epilogue, int splits, int point, float act_pos, float act_neg,
+                            hipStream_t stream) {
+    FSIE_REQUIRE(FSIE_POINT_KNOWN(point) && (point == FSIE_POINT_NONE || (epilogue == 0 && splits == 1 && !out_f32)),
+                 "gemm_mfma_skinny: an activation of the product (%d) goes with a bfloat16 result in one slice", point);
     FSIE_REQUIRE(splits >= 1 && splits <= FSIE_GEMM_MAX_SPLITS, "gemm_mfma_skinny: splits must be 1..%d, got %d",
                  FSIE_GEMM_MAX_SPLITS, splits);
     FSIE_REQUIRE(splits == 1 || (epilogue == 0 && !bias && out_f32),
@@ -60,9 +62,22 @@ extern "C" int fsie_gemm_mfma_skinny(const void* x, const void* w, const float* 
     }
     if (mt * blocks > 4 && waves > 8) waves = 8;  // LDS of the reduction
     fsie_mm::Call call{x, w, bias, y, M, N, K, splits, stream, fsie_mm::RopeArgs{}};
-    call.act = epilogue == 3 ? FSIE_ACT_RELU : (epilogue == 2 ? FSIE_ACT_GELU_TANH : FSIE_ACT_SILU);
+    call.act_pos = act_pos, call.act_neg = act_neg;
+    call.act = epilogue == 0 ? point : epilogue == 3 ? FSIE_ACT_RELU : (epilogue == 2 ? FSIE_ACT_GELU_TANH : FSIE_ACT_SILU);
     if (epilogue != 0) return fsie_mm::launch_swiglu(blocks, waves, call);
     return out_f32 ? fsie_mm::launch_f32(mt, blocks, waves, call) : fsie_mm::launch_bf16(blocks, waves, call);
+}
+
+extern "C" int fsie_gemm_mfma_skinny(const void* x, const void* w, const float* bias, void* y, int M, int N, int K,
+                                     int out_f32, int waves, int blocks, int epilogue, int splits,
+                                     hipStream_t stream) {
+    return gemm_mfma_skinny(x, w, bias, y, M, N, K, out_f32, waves, blocks, epilogue, splits, FSIE_POINT_NONE, 0.f, 0.f, stream);
+}
+
+// y = act(d (+ bias)) in bfloat16, act a FsiePointAct with its constants: the same kernel's plain epilogue.
+extern "C" int fsie_gemm_mfma_skinny_act(const void* x, const void* w, const float* bias, void* y, int M, int N, int K,
+                                         int waves, int blocks, int act, float act_pos, float act_neg, hipStream_t stream) {
+    return gemm_mfma_skinny(x, w, bias, y, M, N, K, 0, waves, blocks, 0, 1, act, act_pos, act_neg, stream);
 }
 
 // The fused q/k/v projection of an attention layer with the position encoding in its epilogue:

@@ -72,7 +72,7 @@ __device__ __forceinline__ void rotation(double pos, double inv_freq, float* c, 
 template <int MT, int NB, int WAVES, typename OutT, int EPI>
 __global__ __launch_bounds__(WAVES * FSIE_WAVE) void gemm_mfma_skinny_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, const float* __restrict__ bias,
-    OutT* __restrict__ y, int M, int N, int K, int k_slice, RopeArgs rope, int act) {
+    OutT* __restrict__ y, int M, int N, int K, int k_slice, RopeArgs rope, int act, float act_pos, float act_neg) {
     constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     __shared__ float red[WAVES > 1 ? (WAVES - 1) * NB * MT * FSIE_WAVE * 4 : 1];
     const int lane = threadIdx.x & (FSIE_WAVE - 1);
@@ -291,7 +291,8 @@ __global__ __launch_bounds__(WAVES * FSIE_WAVE) void gemm_mfma_skinny_kernel(
             for (int r = 0; r < 4; ++r) {
                 const int nn = n0 + nb * 16 + kg * 4 + r;
                 if (nn < N) {
-                    const float v = bias ? acc[nb][t][r] + bias[nn] : acc[nb][t][r];
+                    float v = bias ? acc[nb][t][r] + bias[nn] : acc[nb][t][r];
+                    if constexpr (EPI == EPI_PLAIN && sizeof(OutT) == 2) v = point_act(v, act, act_pos, act_neg);
                     y[static_cast<int64_t>(m) * N + nn] = from_float<OutT>(v);
                 }
             }
@@ -307,7 +308,8 @@ struct Call {
     int splits;  // slices of K, each a workgroup row of its own (partial sums out) when > 1
     hipStream_t stream;
     RopeArgs rope;
-    int act = 0;  // EPI_SWIGLU: the gate's activation (FsieGateAct)
+    int act = 0;  // EPI_SWIGLU: the gate's activation (FsieGateAct); EPI_PLAIN with a bfloat16 result: FsiePointAct
+    float act_pos = 0.f, act_neg = 0.f;  // its constants
 };
 
 template <int MT, int NB, int WAVES, typename OutT, int EPI>
@@ -318,7 +320,7 @@ int launch(const Call& c) {
     const dim3 grid(groups, static_cast<unsigned>(c.splits > 1 ? c.splits : 1));
     gemm_mfma_skinny_kernel<MT, NB, WAVES, OutT, EPI><<<grid, WAVES * FSIE_WAVE, 0, c.stream>>>(
         static_cast<const bf16_t*>(c.x), static_cast<const bf16_t*>(c.w), c.bias, static_cast<OutT*>(c.y), c.M, c.N,
-        c.K, k_slice, c.rope, c.act);
+        c.K, k_slice, c.rope, c.act, c.act_pos, c.act_neg);
     FSIE_CHECK_LAUNCH("gemm_mfma_skinny");
     return 0;
 }

@@ -10,14 +10,15 @@ namespace {
 constexpr int kThreads = 256;
 
 // One block per output row r; source row = rows ? rows[r] : r.
-//   y = delta[row]                          (one array of T, or the sum in order of n_parts float32 arrays)
+//   y = delta[row] (+ delta_bias)           (one array of T, or the sum in order of n_parts float32 arrays)
 //   d = y * rsqrt(mean(y^2) + post_eps) * post_weight
 //   v = residual[row] + d;                  if write_back: residual[row] = v
 //   out[r] = v * rsqrt(mean(v^2) + eps) * weight
 // The row is kept in LDS between the passes (hidden floats).
 template <typename T>
 __global__ __launch_bounds__(kThreads) void sandwich_norm_kernel(
-    float* __restrict__ residual, const T* __restrict__ delta, const float* __restrict__ post_weight, float post_eps,
+    float* __restrict__ residual, const T* __restrict__ delta, const float* __restrict__ delta_bias,
+    const float* __restrict__ post_weight, float post_eps,
     const float* __restrict__ weight, float eps, T* __restrict__ out, const int32_t* __restrict__ rows, int hidden,
     int write_back, int n_parts, int64_t part_stride) {
     extern __shared__ float row_buf[];
@@ -36,6 +37,7 @@ __global__ __launch_bounds__(kThreads) void sandwich_norm_kernel(
             y = 0.f;
             for (int s = 0; s < n_parts; ++s) y += parts[s * part_stride + j];
         }
+        if (delta_bias) y += delta_bias[j];
         row_buf[j] = y;
         sum_sq += y * y;
     }
@@ -73,7 +75,8 @@ __device__ __forceinline__ void store4(bf16_t* p, float4 v) {
 // anything waits.  Places past the end read the last quad again and are masked out of sums and stores.
 template <typename T, int ITERS, int THREADS>
 __global__ __launch_bounds__(THREADS) void sandwich_norm_vec_kernel(
-    float* __restrict__ residual, const T* __restrict__ delta, const float* __restrict__ post_weight, float post_eps,
+    float* __restrict__ residual, const T* __restrict__ delta, const float* __restrict__ delta_bias,
+    const float* __restrict__ post_weight, float post_eps,
     const float* __restrict__ weight, float eps, T* __restrict__ out, const int32_t* __restrict__ rows, int hidden,
     int write_back, int n_parts, int64_t part_stride) {
     __shared__ float scratch[16];
@@ -99,6 +102,10 @@ __global__ __launch_bounds__(THREADS) void sandwich_norm_vec_kernel(
                 a.x += p.x, a.y += p.y, a.z += p.z, a.w += p.w;
             }
             y[it] = a;
+        }
+        if (delta_bias) {
+            const float4 b = load4(delta_bias + j);
+            y[it].x += b.x, y[it].y += b.y, y[it].z += b.z, y[it].w += b.w;
         }
     }
     float sum_sq = 0.f;
@@ -177,9 +184,10 @@ __global__ void softcap_kernel(float* __restrict__ x, int64_t n, float cap, floa
 // The norm of a sublayer's output, the residual sum and the next norm in one pass (see the kernel).
 // delta: [total_rows][hidden] of the activations' type, or with n_parts > 0 that many float32 arrays
 // [total_rows][hidden] one after the other.  rows (or null): the n_rows source rows to work on.
-extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const float* post_weight, float post_eps,
-                                  const float* weight, float eps, void* out, const int32_t* rows, int n_rows, int hidden,
-                                  int dtype, int write_back, int n_parts, int total_rows, hipStream_t stream) {
+// delta_bias [hidden] (or null) is added to every row of it.
+extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const float* delta_bias, const float* post_weight,
+                                  float post_eps, const float* weight, float eps, void* out, const int32_t* rows, int n_rows,
+                                  int hidden, int dtype, int write_back, int n_parts, int total_rows, hipStream_t stream) {
     FSIE_REQUIRE(n_rows >= 0 && hidden > 0 && hidden <= 16384, "sandwich_norm: bad sizes rows=%d hidden=%d (at most 16384)",
                  n_rows, hidden);
     FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "sandwich_norm: unknown dtype %d", dtype);
@@ -191,11 +199,12 @@ extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const floa
     const int64_t part_stride = static_cast<int64_t>(total_rows) * hidden;
     const bool aligned = hidden % 4 == 0 && reinterpret_cast<uintptr_t>(residual) % 16 == 0 &&
                          reinterpret_cast<uintptr_t>(delta) % 16 == 0 && reinterpret_cast<uintptr_t>(post_weight) % 16 == 0 &&
+                         reinterpret_cast<uintptr_t>(delta_bias) % 16 == 0 &&
                          reinterpret_cast<uintptr_t>(weight) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
     if (aligned && hidden <= 8192) {
 #define FSIE_SANDWICH(T, ITERS, THREADS)                                                                             \
     sandwich_norm_vec_kernel<T, ITERS, THREADS><<<n_rows, THREADS, 0, stream>>>(                                     \
-        residual, static_cast<const T*>(delta), post_weight, post_eps, weight, eps, static_cast<T*>(out), rows, hidden, \
+        residual, static_cast<const T*>(delta), delta_bias, post_weight, post_eps, weight, eps, static_cast<T*>(out), rows, hidden, \
         write_back, n_parts, part_stride)
 #define FSIE_SANDWICH_BY_SIZE(T)                                                      \
     if (n_rows <= 128 && hidden > 1024) {  /* few rows: more waves a row */           \
@@ -216,11 +225,11 @@ extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const floa
     }
     const size_t lds = sizeof(float) * hidden;
     if (dtype == FSIE_F32) {
-        sandwich_norm_kernel<float><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const float*>(delta), post_weight,
+        sandwich_norm_kernel<float><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const float*>(delta), delta_bias, post_weight,
                                                                      post_eps, weight, eps, static_cast<float*>(out), rows,
                                                                      hidden, write_back, n_parts, part_stride);
     } else {
-        sandwich_norm_kernel<bf16_t><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const bf16_t*>(delta), post_weight,
+        sandwich_norm_kernel<bf16_t><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const bf16_t*>(delta), delta_bias, post_weight,
                                                                       post_eps, weight, eps, static_cast<bf16_t*>(out), rows,
                                                                       hidden, write_back, n_parts, part_stride);
     }

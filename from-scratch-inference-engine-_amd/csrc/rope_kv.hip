@@ -142,6 +142,7 @@ struct Quad<bf16_t> {
 // PARTS: the projection comes as float32 partial sums parts[n_parts][n_tokens][width] of a product
 // whose inner dimension was cut into slices; they are added in the order of the slices, and qkv
 // only receives the q heads (TOK == 1).
+// Without a table (cos_sin null) nothing is rotated: bias and writes only.
 template <typename T, bool HAS_BIAS, int TOK, bool PARTS = false>
 __global__ __launch_bounds__(kThreads) void rope_kv_write_table_kernel(
     T* __restrict__ qkv, const float* __restrict__ cos_sin, const int32_t* __restrict__ slots,
@@ -243,8 +244,11 @@ __global__ __launch_bounds__(kThreads) void rope_kv_write_table_kernel(
         float4 a1 = load4(t, h * head_dim + i), a2 = load4(t, h * head_dim + i + half);
         a1 = float4{a1.x + b1.x, a1.y + b1.y, a1.z + b1.z, a1.w + b1.w};
         a2 = float4{a2.x + b2.x, a2.y + b2.y, a2.z + b2.z, a2.w + b2.w};
-        const float4* cs = reinterpret_cast<const float4*>(cos_sin + static_cast<int64_t>(t) * head_dim);
-        const float4 c01 = cs[i / 2], c23 = cs[i / 2 + 1];  // (cos, sin) of pairs i, i + 1 and i + 2, i + 3
+        float4 c01{1.f, 0.f, 1.f, 0.f}, c23{1.f, 0.f, 1.f, 0.f};  // (cos, sin) of pairs i, i + 1 and i + 2, i + 3
+        if (cos_sin) {
+            const float4* cs = reinterpret_cast<const float4*>(cos_sin + static_cast<int64_t>(t) * head_dim);
+            c01 = cs[i / 2], c23 = cs[i / 2 + 1];
+        }
         const float4 r1{a1.x * c01.x - a2.x * c01.y, a1.y * c01.z - a2.y * c01.w, a1.z * c23.x - a2.z * c23.y,
                         a1.w * c23.z - a2.w * c23.w};
         const float4 r2{a2.x * c01.x + a1.x * c01.y, a2.y * c01.z + a1.y * c01.w, a2.z * c23.x + a1.z * c23.y,
@@ -338,7 +342,7 @@ extern "C" int fsie_rope_kv_write_table(void* qkv, const float* cos_sin, const i
                  "rope_kv_write_table: 1 to %d aligned partial sums, got %d", FSIE_GEMM_MAX_SPLITS, n_parts);
     FSIE_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv > 0, "rope_kv_write_table: bad sizes");
     FSIE_REQUIRE(head_dim > 0 && head_dim % 8 == 0, "rope_kv_write_table: head_dim %d must be a multiple of 8", head_dim);
-    FSIE_REQUIRE(cos_sin && reinterpret_cast<uintptr_t>(cos_sin) % 16 == 0, "rope_kv_write_table: no aligned table");
+    FSIE_REQUIRE(reinterpret_cast<uintptr_t>(cos_sin) % 16 == 0, "rope_kv_write_table: the table must be 16-byte aligned");
     FSIE_REQUIRE(reinterpret_cast<uintptr_t>(qkv) % 16 == 0 && (!bias || reinterpret_cast<uintptr_t>(bias) % 16 == 0) &&
                      (!k_pool || reinterpret_cast<uintptr_t>(k_pool) % 16 == 0),
                  "rope_kv_write_table: operands must be 16-byte aligned");

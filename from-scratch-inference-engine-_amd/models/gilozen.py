@@ -6,12 +6,33 @@ from __future__ import annotations
 from typing import List
 
 from ..config.base import ConfigError
-from ..config.gilozen import GLA, LATENT, GilozenConfig
+from ..config.gilozen import GLA, LATENT, GilozenConfig, GLAConfig
 from ..parts.base import make_part
 from ..parts.embedding import LMHead, TokenEmbedding
 from ..weights.loader import ParamBinding, TensorSpec
 from .registry import register_architecture
 from .spec import LayerCall, ModelSpec, bind
+
+
+def gla_mixer(bindings: List[ParamBinding], i: int, m: GLAConfig, w: int, eps: float):
+    """Layer i's gated linear attention with its tensors ``l<i>.mix.*`` bound (shared by the architectures that have it)."""
+    p = f"l{i}.mix."
+    kw, vw = m.heads * m.dim, m.heads * m.vdim
+    # the rank of the decays' bottleneck is not in config.json: the tensor's shape gives it
+    rank = m.decay_rank
+    if rank is None:
+        raise ConfigError(f"layer {i}: the rank of the decays' bottleneck is neither in config.json (a_rank) nor "
+                          f"known from the checkpoint's tensor {p}a1: load the configuration from the model folder")
+    mixer = make_part("mixer", "gated_linear_attention", hidden_size=w, n_heads=m.heads, key_dim=m.dim,
+                      value_dim=m.vdim, decay_rank=rank, tau=m.tau, norm_eps=eps, gate_activation="silu")
+    bind(bindings, mixer, "qkvg_weight", [TensorSpec(p + "q", (kw, w)), TensorSpec(p + "k", (kw, w)),
+                                          TensorSpec(p + "v", (vw, w)), TensorSpec(p + "g", (vw, w))])
+    bind(bindings, mixer, "a1_weight", [TensorSpec(p + "a1", (rank, w))])
+    bind(bindings, mixer, "a2_weight", [TensorSpec(p + "a2", (kw, rank))])
+    bind(bindings, mixer, "a2_bias", [TensorSpec(p + "a2.b", (kw,), "bias")])
+    bind(bindings, mixer, "norm_weight", [TensorSpec(p + "norm", (m.vdim,), "norm")])
+    bind(bindings, mixer, "o_weight", [TensorSpec(p + "o", (w, vw))])
+    return mixer
 
 
 def build_gilozen(cfg: GilozenConfig) -> ModelSpec:
@@ -55,21 +76,7 @@ def build_gilozen(cfg: GilozenConfig) -> ModelSpec:
             bind(bindings, mixer, "o_weight", [TensorSpec(p + "o", (w, m.heads * m.vdim))])
             schedule.append(LayerCall(i, cache_of=m.kv_from))
         elif layer.kind == GLA:
-            kw, vw = m.heads * m.dim, m.heads * m.vdim
-            # the rank of the decays' bottleneck is not in config.json: the tensor's shape gives it
-            rank = m.decay_rank
-            if rank is None:
-                raise ConfigError(f"layer {i}: the rank of the decays' bottleneck is neither in config.json (a_rank) nor "
-                                  f"known from the checkpoint's tensor {p}a1: load the configuration from the model folder")
-            mixer = make_part("mixer", "gated_linear_attention", hidden_size=w, n_heads=m.heads, key_dim=m.dim,
-                              value_dim=m.vdim, decay_rank=rank, tau=m.tau, norm_eps=eps, gate_activation="silu")
-            bind(bindings, mixer, "qkvg_weight", [TensorSpec(p + "q", (kw, w)), TensorSpec(p + "k", (kw, w)),
-                                                  TensorSpec(p + "v", (vw, w)), TensorSpec(p + "g", (vw, w))])
-            bind(bindings, mixer, "a1_weight", [TensorSpec(p + "a1", (rank, w))])
-            bind(bindings, mixer, "a2_weight", [TensorSpec(p + "a2", (kw, rank))])
-            bind(bindings, mixer, "a2_bias", [TensorSpec(p + "a2.b", (kw,), "bias")])
-            bind(bindings, mixer, "norm_weight", [TensorSpec(p + "norm", (m.vdim,), "norm")])
-            bind(bindings, mixer, "o_weight", [TensorSpec(p + "o", (w, vw))])
+            mixer = gla_mixer(bindings, i, m, w, eps)
             schedule.append(LayerCall(i))
         else:  # pragma: no cover - the configuration has refused it
             raise ValueError(layer.kind)

@@ -60,8 +60,11 @@ def _ptr(t: Optional[torch.Tensor]) -> Optional[int]:
     return None if t is None else t.data_ptr()
 
 
-def embedding(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor] = None, scale: float = 1.0) -> torch.Tensor:
-    """float32 rows of ``table`` [V, H] at ``ids`` (int32 [T]), times ``scale``.  The caller has checked the ids."""
+def embedding(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor] = None, scale: float = 1.0,
+              pos_table: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """float32 rows of ``table`` [V, H] at ``ids`` (int32 [T]), times ``scale``, plus the rows of ``pos_table`` [P, H] at
+    ``positions`` (int32 [T]; both or neither).  The caller has checked ids and positions (a row that does not exist
+    counts as zeros)."""
     _need(table, "embedding table", ndim=2)
     _need(ids, "embedding ids", dtype=torch.int32, ndim=1)
     v, h = table.shape
@@ -69,8 +72,16 @@ def embedding(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor
     if out is None:
         out = torch.empty((t, h), dtype=torch.float32, device=table.device)
     _need(out, "embedding out", dtype=torch.float32, shape=(t, h))
+    n_positions = 0
+    if pos_table is not None:
+        _need(pos_table, "embedding pos_table", dtype=table.dtype, ndim=2)
+        _need(positions, "embedding positions", dtype=torch.int32, shape=(t,))
+        n_positions = pos_table.shape[0]
+        if pos_table.shape[1] != h:
+            raise KernelError(f"embedding: position rows of {pos_table.shape[1]} values beside token rows of {h}")
     check(load().fsie_embedding(table.data_ptr(), dtype_code(table.dtype), ids.data_ptr(), out.data_ptr(),
-                                t, h, v, float(scale), _stream()))
+                                t, h, v, float(scale), _ptr(pos_table), _ptr(positions) if pos_table is not None else None,
+                                n_positions, _stream()))
     return out
 
 
@@ -203,9 +214,49 @@ def bias_add(y: torch.Tensor, bias: torch.Tensor) -> torch.Tensor:
     return y
 
 
-def sum_round(parts: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+POINT_ACTS = {"none": 0, "xielu": 1}  # activations of one value (no gate) that the kernels know
+
+
+class PointAct:
+    """An activation of single values with its two constants: "xielu" is z / 2 plus ``pos`` z^2 above zero and
+    ``neg`` (exp(z) - 1 - z) below it."""
+
+    __slots__ = ("code", "pos", "neg")
+
+    def __init__(self, name: str, pos: float = 0.0, neg: float = 0.0):
+        if name not in POINT_ACTS:
+            raise KernelError(f"unknown activation '{name}' (known: {sorted(POINT_ACTS)})")
+        self.code, self.pos, self.neg = POINT_ACTS[name], float(pos), float(neg)
+
+
+NO_ACT = PointAct("none")
+
+
+def bias_act(x: torch.Tensor, bias: Optional[torch.Tensor], act: PointAct, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """act(x + bias) for x [T, N] and a float32 bias [N] (or None), in x's type; ``out`` may be ``x``."""
+    _need(x, "bias_act x", ndim=2)
+    if bias is not None:
+        _need(bias, "bias_act bias", dtype=torch.float32, shape=(x.shape[1],))
+    if out is None:
+        out = torch.empty_like(x)
+    _need(out, "bias_act out", dtype=x.dtype, shape=tuple(x.shape))
+    check(load().fsie_bias_act(x.data_ptr(), _ptr(bias), out.data_ptr(), x.shape[0], x.shape[1], dtype_code(x.dtype),
+                               act.code, act.pos, act.neg, _stream()))
+    return out
+
+
+def query_temperature(positions: torch.Tensor, coef: float, every: float) -> torch.Tensor:
+    """float32 [T]: 1 + coef ln(floor((p + 1) / every) + 1) for the positions p (int32 [T])."""
+    _need(positions, "query_temperature positions", dtype=torch.int32, ndim=1)
+    out = torch.empty(positions.shape, dtype=torch.float32, device=positions.device)
+    check(load().fsie_query_temperature(positions.data_ptr(), positions.shape[0], float(coef), float(every), out.data_ptr(),
+                                        _stream()))
+    return out
+
+
+def sum_round(parts: torch.Tensor, bias: Optional[torch.Tensor] = None, act: PointAct = NO_ACT) -> torch.Tensor:
     """bfloat16 [M, N] from float32 partial sums [S, M, N] (or one plane [M, N]): added in their order, plus ``bias``
-    (float32 [N]), rounded once.  N a multiple of 4."""
+    (float32 [N]), through ``act``, rounded once.  N a multiple of 4."""
     if parts.ndim == 2:
         parts = parts.unsqueeze(0)
     _need(parts, "sum_round parts", dtype=torch.float32, ndim=3)
@@ -215,7 +266,7 @@ def sum_round(parts: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch
     if bias is not None:
         _need(bias, "sum_round bias", dtype=torch.float32, shape=(n,))
     y = torch.empty((m, n), dtype=torch.bfloat16, device=parts.device)
-    check(load().fsie_sum_round(parts.data_ptr(), s, _ptr(bias), y.data_ptr(), m, n, _stream()))
+    check(load().fsie_sum_round(parts.data_ptr(), s, _ptr(bias), y.data_ptr(), m, n, act.code, act.pos, act.neg, _stream()))
     return y
 
 
@@ -223,7 +274,8 @@ def rope_kv_write(qkv: torch.Tensor, positions: torch.Tensor, n_heads: int, n_kv
                   inv_freq: Optional[torch.Tensor], slots: Optional[torch.Tensor] = None,
                   k_pool: Optional[torch.Tensor] = None, v_pool: Optional[torch.Tensor] = None,
                   page_size: int = 0, bias: Optional[torch.Tensor] = None,
-                  cos_sin: Optional[torch.Tensor] = None, parts: Optional[torch.Tensor] = None) -> torch.Tensor:
+                  cos_sin: Optional[torch.Tensor] = None, parts: Optional[torch.Tensor] = None,
+                  by_rows: bool = False) -> torch.Tensor:
     """Rotate the q and k heads of ``qkv`` [T, (n_heads + 2 n_kv) head_dim] in place by the angles
     ``positions * inv_freq`` (float64 table of rotary_dim/2 entries; ``None`` = no rotation) and
     copy k and v to the cache slots ``slots`` (int32 [T], negative = not stored) of the pools: keys
@@ -231,7 +283,9 @@ def rope_kv_write(qkv: torch.Tensor, positions: torch.Tensor, n_heads: int, n_kv
     (``rope_table`` of these positions and frequencies): where the whole head is rotated and
     head_dim is a multiple of 8, the kernel reads the angles' cosines and sines there; the table
     alone, without ``inv_freq``, says that the whole head is rotated by it.
-    ``parts`` (float32 [S, T, width], only with ``cos_sin``): the projection as the partial sums of a
+    ``by_rows=True`` (head_dim a multiple of 8, no ``inv_freq``): the table's kernel also where there is no table; it then
+    adds the bias and writes, and rotates nothing.
+    ``parts`` (float32 [S, T, width], only with ``cos_sin`` or ``by_rows``): the projection as the partial sums of a
     product cut along its inner dimension; they are added in order, ``qkv`` is then only written: its
     q columns get the rotated q heads, k and v go to the pools alone."""
     _need(qkv, "qkv", ndim=2)
@@ -247,6 +301,10 @@ def rope_kv_write(qkv: torch.Tensor, positions: torch.Tensor, n_heads: int, n_kv
         if head_dim % 8:
             raise KernelError("rope_kv_write: a table of cosines and sines alone needs a head of a multiple of 8 dimensions")
         rotary_dim = head_dim
+    elif by_rows:
+        if head_dim % 8:
+            raise KernelError("rope_kv_write: whole rows at a time need a head of a multiple of 8 dimensions")
+        rotary_dim = head_dim
     if bias is not None:
         _need(bias, "qkv bias", dtype=torch.float32, shape=(qkv.shape[1],))
     pool_slots = 0
@@ -261,16 +319,17 @@ def rope_kv_write(qkv: torch.Tensor, positions: torch.Tensor, n_heads: int, n_kv
         pool_slots = k_pool.shape[0] * page_size
     n_parts = 0
     if parts is not None:
-        if cos_sin is None or rotary_dim != head_dim or head_dim % 8:
+        if (cos_sin is None and not by_rows) or rotary_dim != head_dim or head_dim % 8:
             raise KernelError("rope_kv_write: partial sums need the table of cosines and sines and a whole head "
                               "of a multiple of 8 dimensions rotated")
         n_parts = parts.shape[0] if parts.dim() == 3 else 0
         _need(parts, "qkv partial sums", dtype=torch.float32, shape=(n_parts, t, qkv.shape[1]))
         if not 1 <= n_parts <= GEMM_MAX_SPLITS:
             raise KernelError(f"rope_kv_write: {n_parts} partial sums; 1 to {GEMM_MAX_SPLITS} are taken")
-    if cos_sin is not None and rotary_dim == head_dim and head_dim % 8 == 0:
-        _need(cos_sin, "cos_sin", dtype=torch.float32, shape=(t, head_dim // 2, 2))
-        check(load().fsie_rope_kv_write_table(qkv.data_ptr(), cos_sin.data_ptr(), _ptr(slots), _ptr(bias),
+    if (cos_sin is not None or (by_rows and inv_freq is None)) and rotary_dim == head_dim and head_dim % 8 == 0:
+        if cos_sin is not None:
+            _need(cos_sin, "cos_sin", dtype=torch.float32, shape=(t, head_dim // 2, 2))
+        check(load().fsie_rope_kv_write_table(qkv.data_ptr(), _ptr(cos_sin), _ptr(slots), _ptr(bias),
                                               _ptr(k_pool), _ptr(v_pool), t, n_heads, n_kv, head_dim, page_size,
                                               pool_slots, dtype_code(qkv.dtype), _ptr(parts), n_parts, _stream()))
         return qkv
@@ -362,6 +421,24 @@ def gemm_mfma_skinny(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch
     return out
 
 
+def gemm_mfma_skinny_act(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], act: PointAct,
+                         waves: int = 0, blocks: int = 0) -> torch.Tensor:
+    """act(x . weight^T + bias) [M, N] in bfloat16 by the few-rows product, the activation in its epilogue: up to 16 rows,
+    K a multiple of 8."""
+    _need(x, "gemm x", dtype=torch.bfloat16, ndim=2)
+    _need(weight, "gemm weight", dtype=torch.bfloat16, ndim=2)
+    m, k = x.shape
+    n = weight.shape[0]
+    if weight.shape[1] != k:
+        raise KernelError(f"gemm: weight inner size {weight.shape[1]} does not match x's {k}")
+    if bias is not None:
+        _need(bias, "gemm bias", dtype=torch.float32, shape=(n,))
+    out = torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
+    check(load().fsie_gemm_mfma_skinny_act(x.data_ptr(), weight.data_ptr(), _ptr(bias), out.data_ptr(), m, n, k, waves,
+                                           blocks, act.code, act.pos, act.neg, _stream()))
+    return out
+
+
 class FragmentOrdered:
     """The copy of a bfloat16 matrix [rows, cols] in the order of the matrix instruction's A
     fragments (``fragment_order``): the 64 16-byte units of a block of 16 rows and 32 columns lie
@@ -436,6 +513,27 @@ def gemm_mfma_wide_swiglu(x: torch.Tensor, weight: torch.Tensor, waves: int = 0,
     check(load().fsie_gemm_mfma_wide_gated(x.data_ptr(), wptr, out.data_ptr(), m, n, k, waves, blocks, frags,
                                            gate_act_code(act), _stream()))
     return out
+
+
+def gemm_mfma_wide_act(x: torch.Tensor, weight, bias: Optional[torch.Tensor], act: PointAct, waves: int = 0,
+                       blocks: int = 0) -> torch.Tensor:
+    """act(x . weight^T + bias) [M, N] in bfloat16 by the kernel that shares x through LDS, the activation in its epilogue
+    (``weight`` or its ``FragmentOrdered`` copy): N a multiple of 4, K of 128, rows as ``gemm_mfma_wide_act_takes`` says."""
+    _need(x, "gemm x", dtype=torch.bfloat16, ndim=2)
+    m, k = x.shape
+    wptr, n, frags = _wide_weight(weight, k)
+    if bias is not None:
+        _need(bias, "gemm bias", dtype=torch.float32, shape=(n,))
+    out = torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
+    check(load().fsie_gemm_mfma_wide_act(x.data_ptr(), wptr, _ptr(bias), out.data_ptr(), m, n, k, waves, blocks, frags,
+                                         act.code, act.pos, act.neg, _stream()))
+    return out
+
+
+def gemm_mfma_wide_act_takes(m: int, weight) -> bool:
+    """Whether ``gemm_mfma_wide_act`` takes ``m`` rows against this weight."""
+    n, k = weight.shape
+    return bool(load().fsie_gemm_mfma_wide_act_takes(int(m), int(n), int(k), int(isinstance(weight, FragmentOrdered))))
 
 
 def gemm_mfma_wide_best_splits(m: int, n: int, k: int) -> int:
@@ -533,8 +631,12 @@ def attention_scalar(q: torch.Tensor, q_stride: int, k_pool: torch.Tensor, v_poo
                      block_tables: torch.Tensor, items: torch.Tensor, n_items: int, out: torch.Tensor,
                      partials: Optional[torch.Tensor], n_heads: int, n_kv: int, head_dim: int,
                      window: Optional[int], scale: float, n_query_rows: int,
-                     sinks: Optional[torch.Tensor] = None, softcap: float = 0.0, pooled=None) -> torch.Tensor:
-    """Attention of the work items over the paged cache (float32 arithmetic).  ``sinks`` (float32 [n_heads],
+                     sinks: Optional[torch.Tensor] = None, softcap: float = 0.0, pooled=None,
+                     slopes: Optional[torch.Tensor] = None, row_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Attention of the work items over the paged cache (float32 arithmetic).  ``slopes`` (float32 [n_heads], here and
+    in the other attention functions): slopes[h] (query position - key position) is taken off head h's scores, behind
+    scale and cap.  ``row_scale`` (float32, one a row of q, here and in the others): a factor on all scores of a row,
+    before the cap.  ``sinks`` (float32 [n_heads],
     here and in the other attention functions): exp(sinks[h]) is one more term of the denominator of
     head h's softmax, with no key and no value.  ``pooled`` = (k_pool, v_pool, block_tables, block_tokens) of the
     pools of pooled blocks (one mean key and value for every ``block_tokens`` positions): items flagged
@@ -571,7 +673,8 @@ def attention_scalar(q: torch.Tensor, q_stride: int, k_pool: torch.Tensor, v_poo
                                        block_tables.data_ptr(), block_tables.shape[1], items.data_ptr(),
                                        n_items, out.data_ptr(), _ptr(partials), n_heads, n_kv, head_dim,
                                        page_size, int(window or 0), float(scale), dtype_code(q.dtype),
-                                       _sinks_ptr(sinks, n_heads), float(softcap or 0.0), *pooled_args, _stream()))
+                                       _sinks_ptr(sinks, n_heads), float(softcap or 0.0), *pooled_args,
+                                       *_bias_ptrs(slopes, row_scale, n_heads, n_query_rows), _stream()))
     return out
 
 
@@ -635,7 +738,8 @@ def attention_mfma(q: torch.Tensor, q_stride: int, k_pool: torch.Tensor, v_pool:
                    block_tables: torch.Tensor, items: torch.Tensor, n_items: int, out: torch.Tensor,
                    partials: Optional[torch.Tensor], n_heads: int, n_kv: int, head_dim: int,
                    window: Optional[int], scale: float, n_query_rows: int, large: bool, waves: int = 1,
-                   sinks: Optional[torch.Tensor] = None, softcap: float = 0.0) -> torch.Tensor:
+                   sinks: Optional[torch.Tensor] = None, softcap: float = 0.0, slopes: Optional[torch.Tensor] = None,
+                   row_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of the work items over the paged cache on the matrix cores (bfloat16; head_dim a
     multiple of 16; page size a multiple of 4).  ``items`` may be a view into a longer table.
     ``waves`` waves of a workgroup split each item's keys and combine inside the workgroup."""
@@ -659,7 +763,8 @@ def attention_mfma(q: torch.Tensor, q_stride: int, k_pool: torch.Tensor, v_pool:
                                      block_tables.data_ptr(), block_tables.shape[1], items.data_ptr(), n_items,
                                      out.data_ptr(), _ptr(partials), n_heads, n_kv, head_dim, page_size,
                                      int(window or 0), float(scale), int(large), int(waves),
-                                     _sinks_ptr(sinks, n_heads), float(softcap or 0.0), _stream()))
+                                     _sinks_ptr(sinks, n_heads), float(softcap or 0.0),
+                                     *_bias_ptrs(slopes, row_scale, n_heads, n_query_rows), _stream()))
     return out
 
 
@@ -668,13 +773,14 @@ def attention_mfma_qkv_ok(head_dim: int, page_size: int) -> bool:
     return bool(load().fsie_attention_mfma_qkv_ok(head_dim, page_size))
 
 
-def attention_mfma_qkv(sums: torch.Tensor, bias: Optional[torch.Tensor], cos_sin: torch.Tensor, slots: torch.Tensor,
+def attention_mfma_qkv(sums: torch.Tensor, bias: Optional[torch.Tensor], cos_sin: Optional[torch.Tensor], slots: torch.Tensor,
                        k_pool: torch.Tensor, v_pool: torch.Tensor, block_tables: torch.Tensor, items: torch.Tensor,
                        n_items: int, out: torch.Tensor, partials: Optional[torch.Tensor], n_heads: int, n_kv: int,
-                       head_dim: int, window: Optional[int], scale: float, waves: int = 1) -> torch.Tensor:
+                       head_dim: int, window: Optional[int], scale: float, waves: int = 1,
+                       slopes: Optional[torch.Tensor] = None, row_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of a step of one token a request (every item: one query row a head) from the q/k/v
     product's float32 partial sums [S, T, (heads + 2 kv heads) head_dim]: the kernel adds them up, adds
-    ``bias``, rotates queries and keys by ``cos_sin`` [T, head_dim / 2, 2], scores each request's new key
+    ``bias``, rotates queries and keys by ``cos_sin`` [T, head_dim / 2, 2] (None: no rotation), scores each request's new key
     from registers and writes it and the value to ``slots[t]`` of the pools (negative: nowhere)."""
     width = (n_heads + 2 * n_kv) * head_dim
     _need(sums, "q/k/v sums", dtype=torch.float32, ndim=3)
@@ -683,9 +789,10 @@ def attention_mfma_qkv(sums: torch.Tensor, bias: Optional[torch.Tensor], cos_sin
         raise KernelError(f"q/k/v sums: shape {tuple(sums.shape)} does not hold rows of {width}")
     if bias is not None:
         _need(bias, "q/k/v bias", dtype=torch.float32, shape=(width,))
-    _need(cos_sin, "cos_sin", dtype=torch.float32)
-    if cos_sin.numel() != t * head_dim:
-        raise KernelError(f"cos_sin: {cos_sin.numel()} values for {t} tokens of head_dim {head_dim}")
+    if cos_sin is not None:
+        _need(cos_sin, "cos_sin", dtype=torch.float32)
+        if cos_sin.numel() != t * head_dim:
+            raise KernelError(f"cos_sin: {cos_sin.numel()} values for {t} tokens of head_dim {head_dim}")
     _need(slots, "slots", dtype=torch.int32, shape=(t,))
     _need(k_pool, "k_pool", dtype=torch.bfloat16, ndim=4)
     _need(v_pool, "v_pool", dtype=torch.bfloat16,
@@ -700,11 +807,12 @@ def attention_mfma_qkv(sums: torch.Tensor, bias: Optional[torch.Tensor], cos_sin
         raise KernelError(f"k_pool: shape {tuple(k_pool.shape)} does not match kv heads {n_kv}, head_dim {head_dim}")
     if partials is not None:
         _need(partials, "attention partials", dtype=torch.float32, ndim=1)
-    check(load().fsie_attention_mfma_qkv(sums.data_ptr(), n_parts, t, _ptr(bias), cos_sin.data_ptr(), slots.data_ptr(),
+    check(load().fsie_attention_mfma_qkv(sums.data_ptr(), n_parts, t, _ptr(bias), _ptr(cos_sin), slots.data_ptr(),
                                          k_pool.data_ptr(), v_pool.data_ptr(), pages * page_size,
                                          block_tables.data_ptr(), block_tables.shape[1], items.data_ptr(), n_items,
                                          out.data_ptr(), _ptr(partials), n_heads, n_kv, head_dim, page_size,
-                                         int(window or 0), float(scale), int(waves), _stream()))
+                                         int(window or 0), float(scale), int(waves),
+                                         *_bias_ptrs(slopes, row_scale, n_heads, t), _stream()))
     return out
 
 
@@ -716,7 +824,8 @@ def attention_mfma_lds_ok(head_dim: int, page_size: int) -> bool:
 def attention_mfma_lds(q: torch.Tensor, q_stride: int, k_pool: torch.Tensor, v_pool: torch.Tensor,
                        block_tables: torch.Tensor, items: torch.Tensor, groups: torch.Tensor, n_groups: int,
                        out: torch.Tensor, n_heads: int, n_kv: int, head_dim: int, window: Optional[int], scale: float,
-                       n_query_rows: int, sinks: Optional[torch.Tensor] = None, softcap: float = 0.0) -> torch.Tensor:
+                       n_query_rows: int, sinks: Optional[torch.Tensor] = None, softcap: float = 0.0,
+                       slopes: Optional[torch.Tensor] = None, row_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of large work items (long portions) with the keys and values of a block staged in
     LDS for four tiles at once.  ``groups`` int32 [n, 2]: index in ``items`` of a group's first
     tile and its number of tiles (1..4, consecutive tiles of one request)."""
@@ -739,7 +848,8 @@ def attention_mfma_lds(q: torch.Tensor, q_stride: int, k_pool: torch.Tensor, v_p
                                          block_tables.data_ptr(), block_tables.shape[1], items.data_ptr(),
                                          groups.data_ptr(), n_groups, out.data_ptr(), n_heads, n_kv, head_dim,
                                          page_size, int(window or 0), float(scale), _sinks_ptr(sinks, n_heads),
-                                         float(softcap or 0.0), _stream()))
+                                         float(softcap or 0.0), *_bias_ptrs(slopes, row_scale, n_heads, n_query_rows),
+                                         _stream()))
     return out
 
 
@@ -748,6 +858,14 @@ def _sinks_ptr(sinks: Optional[torch.Tensor], n_heads: int) -> Optional[int]:
         return None
     _need(sinks, "attention sinks", dtype=torch.float32, shape=(n_heads,))
     return sinks.data_ptr()
+
+
+def _bias_ptrs(slopes: Optional[torch.Tensor], row_scale: Optional[torch.Tensor], n_heads: int, n_rows: int):
+    if slopes is not None:
+        _need(slopes, "attention slopes", dtype=torch.float32, shape=(n_heads,))
+    if row_scale is not None:
+        _need(row_scale, "attention row_scale", dtype=torch.float32, shape=(n_rows,))
+    return _ptr(slopes), _ptr(row_scale)
 
 
 def attention_merge(partials: torch.Tensor, merges: torch.Tensor, n_merges: int, out: torch.Tensor,
@@ -792,15 +910,17 @@ def sample(logits: torch.Tensor, temperature: Optional[torch.Tensor] = None,
 # ---------------------------------------------------------------------------------------------
 def sandwich_norm(residual: torch.Tensor, delta: torch.Tensor, post_weight: torch.Tensor, post_eps: float,
                   weight: Optional[torch.Tensor], eps: float, out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None,
-                  write_back: bool = False) -> torch.Tensor:
+                  write_back: bool = False, delta_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``v = residual + rmsnorm(delta; post_weight, post_eps)``, then ``rmsnorm(v; weight, eps)`` in
-    ``out_dtype``, one pass.  ``delta`` as for ``rmsnorm``; ``write_back`` stores v into ``residual``
+    ``out_dtype``, one pass.  ``delta`` as for ``rmsnorm``, ``delta_bias`` (float32 [H] or None) is added to its rows; ``write_back`` stores v into ``residual``
     (not with ``rows``, which selects the rows to work on)."""
     _need(residual, "sandwich_norm residual", dtype=torch.float32, ndim=2)
     t, h = residual.shape
     if weight is not None:  # (None: the result is v itself, rounded to ``out_dtype``)
         _need(weight, "sandwich_norm weight", dtype=torch.float32, shape=(h,))
     _need(post_weight, "sandwich_norm post weight", dtype=torch.float32, shape=(h,))
+    if delta_bias is not None:
+        _need(delta_bias, "sandwich_norm delta bias", dtype=torch.float32, shape=(h,))
     n_parts = 0
     if delta.ndim == 2 and delta.dtype == torch.float32 and out_dtype != torch.float32:
         delta = delta.unsqueeze(0)  # a float32 delta beside 16-bit activations (the experts' sum): one plane of sums
@@ -818,7 +938,7 @@ def sandwich_norm(residual: torch.Tensor, delta: torch.Tensor, post_weight: torc
         if write_back:
             raise KernelError("sandwich_norm: chosen rows are not written back")
     out = torch.empty((n_rows, h), dtype=out_dtype, device=residual.device)
-    check(load().fsie_sandwich_norm(residual.data_ptr(), delta.data_ptr(), post_weight.data_ptr(), float(post_eps),
+    check(load().fsie_sandwich_norm(residual.data_ptr(), delta.data_ptr(), _ptr(delta_bias), post_weight.data_ptr(), float(post_eps),
                                     _ptr(weight), float(eps), out.data_ptr(), _ptr(rows), n_rows, h,
                                     dtype_code(out_dtype), int(write_back), n_parts, t, _stream()))
     return out

@@ -26,7 +26,7 @@ _SIGNATURES = {
     "fsie_version": ([], c_int),
     "fsie_device_info": ([c_char_p, c_int, ctypes.POINTER(c_int)], c_int),
     "fsie_device_compute_units": ([], c_int),
-    "fsie_embedding": ([_P, c_int, _P, _P, c_int, c_int, c_int, c_float, _P], c_int),
+    "fsie_embedding": ([_P, c_int, _P, _P, c_int, c_int, c_int, c_float, _P, _P, c_int, _P], c_int),
     "fsie_rmsnorm": ([_P, _P, _P, _P, _P, c_int, c_int, c_float, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_rmsnorm_plain": ([_P, c_int64, _P, _P, c_int64, c_int, c_int, c_int, c_float, c_int, _P], c_int),
     "fsie_zero_rows": ([_P, _P, c_int, c_int64, c_int, _P], c_int),
@@ -38,7 +38,9 @@ _SIGNATURES = {
     "fsie_scaled_sum": ([_P, c_float, _P, c_float, _P, c_int64, c_int, _P], c_int),
     "fsie_pool_blocks": ([_P, _P, _P, c_int, c_int, _P, _P, _P, c_int, c_int, _P, c_int, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_bias_add": ([_P, _P, c_int, c_int, c_int, _P], c_int),
-    "fsie_sum_round": ([_P, c_int, _P, _P, c_int, c_int, _P], c_int),
+    "fsie_sum_round": ([_P, c_int, _P, _P, c_int, c_int, c_int, c_float, c_float, _P], c_int),
+    "fsie_bias_act": ([_P, _P, _P, c_int, c_int, c_int, c_int, c_float, c_float, _P], c_int),
+    "fsie_query_temperature": ([_P, c_int, c_double, c_double, _P, _P], c_int),
     "fsie_rope_kv_write": ([_P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int64,
                             c_int, _P], c_int),
     "fsie_rope_kv_write_table": ([_P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int64, c_int, _P, c_int, _P],
@@ -53,20 +55,23 @@ _SIGNATURES = {
     "fsie_gemm_mfma_wide_best_splits": ([c_int, c_int, c_int], c_int),
     "fsie_gemm_mfma_wide": ([_P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_gemm_mfma_wide_swiglu": ([_P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P], c_int),
+    "fsie_gemm_mfma_skinny_act": ([_P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, _P], c_int),
+    "fsie_gemm_mfma_wide_act": ([_P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, _P], c_int),
+    "fsie_gemm_mfma_wide_act_takes": ([c_int, c_int, c_int, c_int], c_int),
     "fsie_gemm_mfma_wide_takes": ([c_int, c_int, c_int, c_int, c_int, c_int], c_int),
     "fsie_fragment_order_size": ([c_int, c_int], c_int64),
     "fsie_fragment_order": ([_P, _P, c_int, c_int, _P], c_int),
     "fsie_attention_scalar": ([_P, c_int64, _P, _P, _P, c_int, _P, c_int, _P, _P, c_int, c_int, c_int,
-                               c_int, c_int, c_float, c_int, _P, c_float, _P, _P, _P, c_int, c_int, c_int, _P], c_int),
+                               c_int, c_int, c_float, c_int, _P, c_float, _P, _P, _P, c_int, c_int, c_int, _P, _P, _P], c_int),
     "fsie_attention_mfma": ([_P, c_int64, _P, _P, _P, c_int, _P, c_int, _P, _P, c_int, c_int, c_int,
-                             c_int, c_int, c_float, c_int, c_int, _P, c_float, _P], c_int),
+                             c_int, c_int, c_float, c_int, c_int, _P, c_float, _P, _P, _P], c_int),
     "fsie_attention_mfma_qkv_ok": ([c_int, c_int], c_int),
     "fsie_attention_mfma_qkv": ([_P, c_int, c_int, _P, _P, _P, _P, _P, c_int64, _P, c_int, _P, c_int, _P, _P, c_int,
-                                 c_int, c_int, c_int, c_int, c_float, c_int, _P], c_int),
+                                 c_int, c_int, c_int, c_int, c_float, c_int, _P, _P, _P], c_int),
     "fsie_attention_mfma_max_waves": ([c_int], c_int),
     "fsie_attention_mfma_lds_ok": ([c_int, c_int], c_int),
     "fsie_attention_mfma_lds": ([_P, c_int64, _P, _P, _P, c_int, _P, _P, c_int, _P, c_int, c_int, c_int, c_int, c_int,
-                                 c_float, _P, c_float, _P], c_int),
+                                 c_float, _P, c_float, _P, _P, _P], c_int),
     "fsie_attention_mfma_tiles": ([c_int, c_int], c_int),
     "fsie_attention_merge": ([_P, _P, c_int, _P, c_int, c_int, c_int, _P, _P], c_int),
     "fsie_attention_scalar_tile_tokens": ([c_int, c_int], c_int),
@@ -75,7 +80,7 @@ _SIGNATURES = {
                                      c_int, c_int, c_int, c_float, c_int, c_int, c_int, _P], c_int),
     "fsie_gated_act": ([_P, _P, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_gemm_mfma_wide_gated": ([_P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P], c_int),
-    "fsie_sandwich_norm": ([_P, _P, _P, c_float, _P, c_float, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P], c_int),
+    "fsie_sandwich_norm": ([_P, _P, _P, _P, c_float, _P, c_float, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_gated_headnorm": ([_P, c_int, _P, c_int64, _P, _P, c_int, c_int, c_int, c_float, c_int, c_int, c_int64, c_float, _P], c_int),
     "fsie_gla_scan_shape": ([c_int, c_int, c_int, ctypes.POINTER(c_int), ctypes.POINTER(c_int), ctypes.POINTER(c_int),
                              ctypes.POINTER(c_int), ctypes.POINTER(c_int64)], c_int),

@@ -3,7 +3,7 @@
 from __future__ import annotations
 
 import math
-from typing import Dict, Optional
+from typing import Dict, Optional, Sequence, Tuple
 
 import numpy as np
 import torch
@@ -459,7 +459,8 @@ class AttentionPlanner:
 
 def paged_attention(q: torch.Tensor, q_stride: int, cache, plan, n_heads: int, n_kv: int, head_dim: int,
                     window: Optional[int], scale: float, n_tokens: int, sinks: Optional[torch.Tensor] = None,
-                    share_keys: bool = True, softcap: Optional[float] = None, pooled=None) -> torch.Tensor:
+                    share_keys: bool = True, softcap: Optional[float] = None, pooled=None,
+                    slopes: Optional[torch.Tensor] = None, row_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal attention of a step's queries over the paged cache, by the work items of ``plan`` (an
     ``AttentionPlanner``'s): [n_tokens, n_heads * head_dim] in the queries' type.  ``q``: rows of ``q_stride``
     values whose first n_heads * head_dim are the heads' queries; the keys and values of the step's own
@@ -467,7 +468,9 @@ def paged_attention(q: torch.Tensor, q_stride: int, cache, plan, n_heads: int, n
     denominator of head h's softmax.  ``softcap`` (a positive number or None): the scaled scores become
     softcap * tanh(score / softcap) before the mask and the softmax.  ``pooled`` = (k_pool, v_pool, block_tables,
     block_tokens): the pools of pooled blocks that items flagged ``ATTN_POOL_WALK`` read beside their keys (a planner
-    with ``pool``).  Every mixer whose cache is pages of keys and values calls this."""
+    with ``pool``).  ``slopes`` (float32 [n_heads] or None): slopes[h] (query position - key position) is taken off head
+    h's scores, behind scale and cap.  ``row_scale`` (float32 [n_tokens] or None): a factor on all scores of a token,
+    before the cap.  Every mixer whose cache is pages of keys and values calls this."""
     cap = float(softcap or 0.0)
     if pooled is not None and plan.mfma and plan.n_pool_items and not plan.n_partial:
         raise RuntimeError("attention: items of pooled blocks without partial records to leave them in")
@@ -476,29 +479,30 @@ def paged_attention(q: torch.Tensor, q_stride: int, cache, plan, n_heads: int, n
     if plan.n_partial:
         partials = torch.empty((plan.n_partial * n_heads * (head_dim + 2),), dtype=torch.float32, device=q.device)
     args = (partials, n_heads, n_kv, head_dim, window, scale, n_tokens)
+    bias = dict(slopes=slopes, row_scale=row_scale)
     if plan.mfma:
         if plan.n_small:
             ops.attention_mfma(q, q_stride, cache.k_pool, cache.v_pool, cache.block_tables, plan.items,
-                               plan.n_small, out, *args, large=False, waves=plan.waves, sinks=sinks, softcap=cap)
+                               plan.n_small, out, *args, large=False, waves=plan.waves, sinks=sinks, softcap=cap, **bias)
         if (plan.n_large and (not plan.n_long or getattr(plan, "long_waves", 4) == 1) and share_keys
                 and ops.attention_mfma_lds_ok(head_dim, cache.page_size)):
             ops.attention_mfma_lds(q, q_stride, cache.k_pool, cache.v_pool, cache.block_tables,
                                    plan.items[plan.n_small:], plan.groups, plan.n_groups, out, n_heads,
-                                   n_kv, head_dim, window, scale, n_tokens, sinks=sinks, softcap=cap)
+                                   n_kv, head_dim, window, scale, n_tokens, sinks=sinks, softcap=cap, **bias)
         elif plan.n_large:
             ops.attention_mfma(q, q_stride, cache.k_pool, cache.v_pool, cache.block_tables,
-                               plan.items[plan.n_small:], plan.n_large, out, *args, large=True, sinks=sinks, softcap=cap)
+                               plan.items[plan.n_small:], plan.n_large, out, *args, large=True, sinks=sinks, softcap=cap, **bias)
         if plan.n_long:
             ops.attention_mfma(q, q_stride, cache.k_pool, cache.v_pool, cache.block_tables,
                                plan.items[plan.n_small + plan.n_large:], plan.n_long, out, *args, large=True,
-                               waves=getattr(plan, "long_waves", 4), sinks=sinks, softcap=cap)
+                               waves=getattr(plan, "long_waves", 4), sinks=sinks, softcap=cap, **bias)
         if pooled is not None and plan.n_pool_items:
             # the pooled blocks of the queries that see any: partial records beside those of their keys
             ops.attention_scalar(q, q_stride, cache.k_pool, cache.v_pool, cache.block_tables, plan.pool_items,
-                                 plan.n_pool_items, out, *args, softcap=cap, pooled=pooled)
+                                 plan.n_pool_items, out, *args, softcap=cap, pooled=pooled, **bias)
     else:
         ops.attention_scalar(q, q_stride, cache.k_pool, cache.v_pool, cache.block_tables, plan.items,
-                             plan.n_small + plan.n_large, out, *args, sinks=sinks, softcap=cap, pooled=pooled)
+                             plan.n_small + plan.n_large, out, *args, sinks=sinks, softcap=cap, pooled=pooled, **bias)
     if plan.n_merges:
         ops.attention_merge(partials, plan.merges, plan.n_merges, out, n_heads, head_dim, sinks=sinks)
     return out
@@ -535,6 +539,10 @@ class GQAttention(Mixer):
     block of ``pool`` positions that lies wholly before its window; the means are kept in pages of their own (an entry a
     block, a second cache need) and made by a kernel from the cached keys and values when a block's last position
     arrives.  ``fused_prep=True`` takes the one-kernel path below also where none of its reasons holds.
+    ``slopes``: a number per query head; slopes[h] (query position - key position) is taken off head h's scores, behind
+    scale and cap (a bias by distance; it needs the position of every key, so not with pooled blocks).
+    ``query_temperature`` = (coef, every): the queries at position p are multiplied by
+    1 + coef ln(floor((p + 1) / every) + 1); the attention kernels take the factor as one number a token, in float32.
     With any of gate, mixed values, another value size or the unit norm, what stands between projection and attention is one kernel
     (``ops.attention_prep``: head norms, rotation of the first ``rotary_dim`` values from the step's table, value
     mixing, gates, cache write) and one after it (``ops.gate_heads``).
@@ -547,7 +555,8 @@ class GQAttention(Mixer):
     kernels do several of these steps at once: for steps of one token a request the attention
     kernel itself finishes the projection's partial sums (bias, rotation, cache write); for up to 16
     rows the projection's epilogue does; for 17 to 128 rows the kernel that writes the cache adds
-    the partial sums up.  With head norms, or an encoding without a table, the steps run one after
+    the partial sums up.  An encoding that leaves q and k alone (``rotates`` False) takes the same kernels, which then
+    rotate nothing.  With head norms, or an encoding without a table, the steps run one after
     the other (projection, bias, norms, ``rotate``, cache write), which every combination can take."""
 
     share_keys = True  # long portions: four tiles of a request share each block of keys through LDS
@@ -567,7 +576,8 @@ class GQAttention(Mixer):
                  o_bias: bool = False, unit_norm_eps: Optional[float] = None, head_temperature: bool = False,
                  softcap: Optional[float] = None, interleaved_pairs: bool = False,
                  value_unit_norm_eps: Optional[float] = None, unit_sink: bool = False, chunk: Optional[int] = None,
-                 pool: Optional[int] = None, fused_prep: bool = False):
+                 pool: Optional[int] = None, fused_prep: bool = False, slopes: Optional[Sequence[float]] = None,
+                 query_temperature: Optional[Tuple[float, float]] = None):
         if n_heads % n_kv_heads:
             raise ValueError(f"attention: heads {n_heads} must be a multiple of kv heads {n_kv_heads}")
         self.value_dim = head_dim if value_dim is None else int(value_dim)
@@ -606,6 +616,13 @@ class GQAttention(Mixer):
         if pool is not None and (pool < 1 or not window or keep_first):
             raise ValueError("attention: pooled blocks are a positive number of positions and go with a plain window")
         self.chunk, self.pool = chunk, pool
+        if slopes is not None and (len(slopes) != n_heads or pool is not None):
+            raise ValueError("attention: slopes are one number a query head and do not go with pooled blocks")
+        self.slopes = None if slopes is None else tuple(float(v) for v in slopes)
+        self._slopes: Optional[torch.Tensor] = None
+        if query_temperature is not None and not float(query_temperature[1]) > 0:
+            raise ValueError(f"attention: the period of the query temperature {query_temperature[1]} must be positive")
+        self.query_temperature = None if query_temperature is None else tuple(float(v) for v in query_temperature)
         self.prepared = (self.has_gate or value_mix is not None or self.value_dim != head_dim or self.unit_norm_eps is not None
                          or self.value_unit_norm_eps is not None or pool is not None or bool(fused_prep) or self.interleaved_pairs)
         if self.prepared:
@@ -674,6 +691,8 @@ class GQAttention(Mixer):
             for norm in {id(n): n for n in (self.q_norm, self.k_norm) if n is not None}.values():
                 norm.weight = norm.weight[order].contiguous()
             self._reordered = True
+        if self.slopes is not None:
+            self._slopes = torch.tensor(self.slopes, dtype=torch.float32, device=device)
         if self.unit_sink:
             self.sink = torch.zeros((self.n_heads,), dtype=torch.float32, device=device)
         if self.unit_norm_eps is not None:
@@ -705,18 +724,31 @@ class GQAttention(Mixer):
         return self._planner
 
     # compute ----------------------------------------------------------------------------
-    def _fused_table(self, ctx) -> Optional[torch.Tensor]:
-        """The rotation as a table, if the mixer's fused kernels may stand for bias + rotate + write:
-        nothing between the projection and the rotation, and an encoding that is such a rotation
-        (or none at all: then the kernels only add the bias and write)."""
-        if self.q_norm is not None or self.k_norm is not None or self.head_dim % 8:
+    def _row_scale(self, ctx) -> Optional[torch.Tensor]:
+        """The step's factors on the scores of its tokens: the same in every layer with these constants, made by the
+        first one that asks."""
+        if self.query_temperature is None:
             return None
-        return self.position.rotation_table(self.head_dim, ctx)
+        key = ("query temperature", *self.query_temperature)
+        if key not in ctx.memo:
+            ctx.memo[key] = ops.query_temperature(ctx.positions, *self.query_temperature)
+        return ctx.memo[key]
 
-    def _from_sums(self, x: torch.Tensor, ctx, cache, plan, table) -> Optional[torch.Tensor]:
+    def _fused_table(self, ctx):
+        """(may fuse, table): whether the mixer's fused kernels may stand for bias + rotate + write (nothing between the
+        projection and the rotation, and an encoding that is such a rotation or none at all: then the kernels only
+        add the bias and write), and the rotation as a table (None: no rotation)."""
+        if self.q_norm is not None or self.k_norm is not None or self.head_dim % 8:
+            return False, None
+        if not self.position.rotates:
+            return True, None
+        table = self.position.rotation_table(self.head_dim, ctx)
+        return table is not None, table
+
+    def _from_sums(self, x: torch.Tensor, ctx, cache, plan, fuse: bool, table) -> Optional[torch.Tensor]:
         """Attention of a step of one token a request straight from the q/k/v product's partial sums
         (None: not such a step, or the kernels do not take the sizes)."""
-        if not (self.finish_qkv_in_attention and self.sink is None and not self.keep_first and self.softcap is None and table is not None and cache.writes and plan.mfma and plan.single
+        if not (self.finish_qkv_in_attention and self.sink is None and not self.keep_first and self.softcap is None and fuse and cache.writes and plan.mfma and plan.single
                 and plan.n_small and not plan.n_large and not plan.n_long and x.dtype == torch.bfloat16
                 and ops.attention_mfma_qkv_ok(self.head_dim, cache.page_size)):
             return None
@@ -730,12 +762,13 @@ class GQAttention(Mixer):
                                    device=x.device)
         ops.attention_mfma_qkv(sums, self.qkv.bias, table, cache.slots, cache.k_pool, cache.v_pool,
                                cache.block_tables, plan.items, plan.n_small, out, partials, self.n_heads, self.n_kv,
-                               self.head_dim, self.window, self.scale, waves=plan.waves)
+                               self.head_dim, self.window, self.scale, waves=plan.waves, slopes=self._slopes,
+                               row_scale=self._row_scale(ctx))
         if plan.n_merges:
             ops.attention_merge(partials, plan.merges, plan.n_merges, out, self.n_heads, self.head_dim)
         return out
 
-    def _project_rotate_store(self, x: torch.Tensor, ctx, cache, table) -> torch.Tensor:
+    def _project_rotate_store(self, x: torch.Tensor, ctx, cache, fuse: bool, table) -> torch.Tensor:
         """q/k/v [T, (heads + 2 kv heads) head_dim] of which attention reads the q columns: projected,
         with the bias, the head norms and the rotation applied, and k and v written into the cache
         (unless this call only reads another call's cache)."""
@@ -743,7 +776,7 @@ class GQAttention(Mixer):
         store = dict(slots=cache.slots, k_pool=cache.k_pool, v_pool=cache.v_pool,
                      page_size=cache.page_size) if cache.writes else {}
         bias = self.qkv.bias
-        if table is not None:
+        if fuse:
             if x.dtype == torch.bfloat16 and 0 < x.shape[0] <= GEMM_MFMA_SKINNY_BEST_M and x.shape[1] % 8 == 0 and hd % 16 == 0:
                 # a few rows of a step that is not one token a request: the projection's own epilogue
                 # adds the bias, rotates and stores
@@ -754,10 +787,10 @@ class GQAttention(Mixer):
                 # 17 to 128 rows: the engine's product in slices of K, added up by the kernel that rotates
                 qkv = torch.empty(sums.shape[1:], dtype=ctx.compute_dtype, device=x.device)
                 return ops.rope_kv_write(qkv, ctx.positions, nh, nkv, hd, None, bias=bias, cos_sin=table,
-                                         parts=sums, **store)
+                                         parts=sums, by_rows=True, **store)
         qkv = self.qkv(x, skip_bias=True)
-        if table is not None:
-            return ops.rope_kv_write(qkv, ctx.positions, nh, nkv, hd, None, bias=bias, cos_sin=table, **store)
+        if fuse:
+            return ops.rope_kv_write(qkv, ctx.positions, nh, nkv, hd, None, bias=bias, cos_sin=table, by_rows=True, **store)
         # one step after the other
         plain_write = not self.position.rotates and self.q_norm is None and self.k_norm is None
         if bias is not None and not plain_write:
@@ -826,7 +859,8 @@ class GQAttention(Mixer):
                                 blocks.block_tables, plan.pool_jobs, plan.n_pool_jobs, self.pool)
             pooled = (blocks.k_pool, blocks.v_pool, blocks.block_tables, self.pool)
         out = paged_attention(q, nh * pd, cache, plan, nh, nkv, pd, self.window, self.scale, x.shape[0], sinks=self.sink,
-                              share_keys=self.share_keys, softcap=self.softcap, pooled=pooled)
+                              share_keys=self.share_keys, softcap=self.softcap, pooled=pooled, slopes=self._slopes,
+                              row_scale=self._row_scale(ctx))
         if heads_out is not None:
             ops.gate_heads(out, pd, vd, nh, gate, out=heads_out, scale=heads_scale)
             return None
@@ -838,11 +872,12 @@ class GQAttention(Mixer):
         plan = ctx.plan(self.planner())
         if self.prepared:
             return self._forward_prepared(x, ctx, cache, plan)
-        table = self._fused_table(ctx)
-        out = self._from_sums(x, ctx, cache, plan, table)
+        fuse, table = self._fused_table(ctx)
+        out = self._from_sums(x, ctx, cache, plan, fuse, table)
         if out is not None:
             return self.o.for_residual(out, ctx)
-        qkv = self._project_rotate_store(x, ctx, cache, table)
+        qkv = self._project_rotate_store(x, ctx, cache, fuse, table)
         out = paged_attention(qkv, qkv.shape[1], cache, plan, self.n_heads, self.n_kv, self.head_dim, self.window,
-                              self.scale, x.shape[0], sinks=self.sink, share_keys=self.share_keys, softcap=self.softcap)
+                              self.scale, x.shape[0], sinks=self.sink, share_keys=self.share_keys, softcap=self.softcap,
+                              slopes=self._slopes, row_scale=self._row_scale(ctx))
         return self.o.for_residual(out, ctx)

@@ -51,10 +51,12 @@ class HiddenState:
     pending delta goes through before it is added (a layer that also norms its sublayers' outputs), or
     None; the norm that folds the delta in applies it in the same pass.  ``delta2``: a second pending delta of
     the same kinds, left by a block whose mixer and feed-forward read the same stream (only norms that set
-    ``adds_two_deltas`` take it; the others refuse).  ``delta_scale``: a factor on the pending deltas when they are
+    ``adds_two_deltas`` take it; the others refuse).  ``delta_bias``: a float32 [H] that belongs to the pending delta (the
+    bias of the product it comes from) and is added to it first, or None (only norms that set ``adds_delta_bias`` take it,
+    together with ``delta_norm``).  ``delta_scale``: a factor on the pending deltas when they are
     added, x += delta_scale * (delta + delta2) (only norms that set ``scales_deltas`` take another value than 1)."""
 
-    __slots__ = ("residual", "delta", "delta_norm", "delta2", "delta_scale")
+    __slots__ = ("residual", "delta", "delta_norm", "delta2", "delta_scale", "delta_bias")
 
     def __init__(self, residual: torch.Tensor, delta: Optional[torch.Tensor] = None, delta_norm=None):
         self.residual = residual
@@ -62,6 +64,7 @@ class HiddenState:
         self.delta_norm = delta_norm
         self.delta2 = None
         self.delta_scale = 1.0
+        self.delta_bias = None
 
 
 class Part:
@@ -117,6 +120,8 @@ class Norm(Part):
     # True if the norm adds a second pending delta (``HiddenState.delta2``) in the same pass, and offers
     # ``pair(hidden, other, out_dtype)``: this norm's and another one's output of the same stream at once
     adds_two_deltas = False
+    # True if the norm adds ``HiddenState.delta_bias`` to a pending delta that comes with a norm of its own
+    adds_delta_bias = False
     # True if the norm multiplies the pending deltas by ``HiddenState.delta_scale`` as it adds them
     scales_deltas = False
 
@@ -149,6 +154,9 @@ class Mixer(Part):
 
 class FeedForward(Part):
     kind = "feed_forward"
+    # a bias (float32 [H]) that belongs to what ``forward`` returns and that the block hands to the norm that adds it
+    # (``HiddenState.delta_bias``); None: what ``forward`` returns is whole
+    residual_bias: Optional[torch.Tensor] = None
 
     def forward(self, x: torch.Tensor, ctx) -> torch.Tensor:
         raise NotImplementedError

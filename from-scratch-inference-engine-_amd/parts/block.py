@@ -9,6 +9,12 @@ import torch
 from .base import Block, Convolution, FeedForward, HiddenState, Mixer, Norm, Part, register_part
 
 
+def _whole_output(ffn: Optional[FeedForward], block: str) -> None:
+    if ffn is not None and getattr(ffn, "defer_bias", False):
+        raise ValueError(f"{block} block: a feed-forward that leaves its last bias to the next norm needs a block that hands "
+                         f"it on (sandwich_norm does)")
+
+
 @register_part("block", "pre_norm")
 class PreNormBlock(Block):
     """x += mixer(norm1(x)); x += ffn(norm2(x))  (src/model/model.cpp:106-139).  The sums are
@@ -18,6 +24,7 @@ class PreNormBlock(Block):
     graph_safe = True
 
     def __init__(self, mixer_norm: Norm, mixer: Mixer, ffn_norm: Norm, ffn: FeedForward):
+        _whole_output(ffn, "pre_norm")
         self.mixer_norm, self.mixer, self.ffn_norm, self.ffn = mixer_norm, mixer, ffn_norm, ffn
 
     def sub_parts(self) -> Dict[str, Part]:
@@ -35,7 +42,8 @@ class SandwichNormBlock(Block):
     """A norm before and after every sublayer: x += post1(mixer(norm1(x))); x += post2(ffn(norm2(x))).
     A sublayer's output stays pending in the hidden state together with its post norm; the norm that reads
     the stream next (this block's second, the next block's first, the model's last) runs the post norm,
-    the sum and itself in one pass.  ``ffn=None``: the layer has no feed-forward (and no norms for it)."""
+    the sum and itself in one pass, with the bias of the feed-forward's last product where that leaves it pending
+    (``FeedForward.residual_bias``).  ``ffn=None``: the layer has no feed-forward (and no norms for it)."""
 
     graph_safe = True
 
@@ -58,6 +66,7 @@ class SandwichNormBlock(Block):
         if self.ffn is not None:
             x = self.ffn_norm(hidden, ctx.compute_dtype)
             hidden.delta, hidden.delta_norm = self.ffn.forward(x, ctx), self.ffn_post_norm
+            hidden.delta_bias = self.ffn.residual_bias
 
 
 @register_part("block", "branch_norm")
@@ -73,6 +82,7 @@ class BranchNormBlock(Block):
                  ffn_post_norm: Optional[Norm] = None):
         if (ffn is None) != (ffn_post_norm is None):
             raise ValueError("branch_norm block: a feed-forward comes with the norm of its output, or neither")
+        _whole_output(ffn, "branch_norm")
         self.reader, self.mixer, self.mixer_post_norm = reader, mixer, mixer_post_norm
         self.ffn, self.ffn_post_norm = ffn, ffn_post_norm
 
@@ -106,6 +116,7 @@ class ParallelBlock(Block):
                  ffn_conv: Optional[Convolution] = None):
         if (ffn is None) != (ffn_norm is None):
             raise ValueError("parallel block: a feed-forward comes with its norm, or neither")
+        _whole_output(ffn, "parallel")
         if ffn is None and ffn_conv is not None:
             raise ValueError("parallel block: a convolution in front of a feed-forward that is not there")
         if not mixer_norm.adds_two_deltas or (ffn_norm is not None and not ffn_norm.adds_two_deltas):

@@ -44,6 +44,31 @@ class TokenEmbedding(Part):
         return self.forward(ctx.token_ids)
 
 
+class PositionedEmbedding(TokenEmbedding):
+    """x[t] = table[ids[t]] * scale + places[position of t]: a learned vector for each of ``n_positions`` positions, added
+    in float32 in the same pass.  Positions are the step's own table, so portions, single tokens and replayed graphs all
+    see them; a request may not grow beyond ``n_positions`` (the step function refuses by the configuration's
+    ``max_positions``)."""
+
+    def __init__(self, vocab_size: int, hidden_size: int, n_positions: int, scale: float = 1.0):
+        super().__init__(vocab_size, hidden_size, scale)
+        if n_positions < 1:
+            raise ValueError(f"positioned embedding: {n_positions} positions")
+        self.n_positions = int(n_positions)
+        self.position_weight = None
+
+    def param_decls(self) -> Dict[str, ParamDecl]:
+        return {"weight": ParamDecl((self.vocab_size, self.hidden_size)),
+                "position_weight": ParamDecl((self.n_positions, self.hidden_size))}
+
+    def forward(self, ids: torch.Tensor) -> torch.Tensor:
+        raise RuntimeError("positioned embedding: the step's positions are needed (embed)")
+
+    def embed(self, ctx, cache) -> torch.Tensor:
+        return ops.embedding(self.weight, ctx.token_ids, scale=self.scale, pos_table=self.position_weight,
+                             positions=ctx.positions)
+
+
 class PairHashEmbedding(TokenEmbedding):
     """x[t] = table[id_t] * scale + pairs[(id_{t-1} * mul_prev + id_t * mul_cur) mod buckets]: a second table of
     ``buckets`` + 1 rows, addressed by a hash of the token and the one before it; a request's first token takes the

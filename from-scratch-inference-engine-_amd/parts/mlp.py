@@ -1,8 +1,9 @@
-"""Dense gated feed-forward."""
+"""Dense feed-forwards, with and without a gate."""
 
 from __future__ import annotations
 
-from typing import Dict
+import math
+from typing import Dict, Optional
 
 import torch
 
@@ -81,3 +82,82 @@ class SwiGLU(FeedForward):
         else:
             act = ops.swiglu(self.gate_up(x), act=self.activation)
         return self.down.for_residual(act, ctx)
+
+
+def _softplus(v: float) -> float:
+    return max(v, 0.0) + math.log1p(math.exp(-abs(v)))
+
+
+@register_part("feed_forward", "plain")
+class PlainFeedForward(FeedForward):
+    """down(act(up(x) + b_up)) + b_down without a gate.  act = xIELU with two learned numbers (p, q) (parameter ``act``):
+    softplus(p) z^2 + z / 2 above zero, (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2 below it; the softpluses are taken
+    once, when the weights are loaded.
+
+    Bias and activation happen in the first product's epilogue for the rows that the engine's own products take, in the
+    kernel that adds up its partial sums, or in one pass of their own behind the library's product.
+    ``defer_bias=True``: the second bias is not added here but left in ``residual_bias`` for the norm that adds this
+    part's output to the stream (``HiddenState.delta_bias``), so that the second product may leave partial sums."""
+
+    graph_safe = True
+
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "xielu", bias: bool = True,
+                 defer_bias: bool = False):
+        if activation != "xielu":
+            raise ValueError(f"feed-forward: unknown activation '{activation}' (xielu)")
+        self.hidden_size, self.intermediate_size = hidden_size, intermediate_size
+        self.has_bias, self.defer_bias = bool(bias), bool(defer_bias) and bool(bias)
+        self.up = Linear(hidden_size, intermediate_size, bias=self.has_bias)
+        self.down = Linear(intermediate_size, hidden_size, bias=self.has_bias and not self.defer_bias)
+        self.act: Optional[torch.Tensor] = None
+        self._act: Optional[ops.PointAct] = None
+
+    def param_decls(self) -> Dict[str, ParamDecl]:
+        decls = {"up_weight": ParamDecl((self.intermediate_size, self.hidden_size)),
+                 "down_weight": ParamDecl((self.hidden_size, self.intermediate_size)),
+                 "act": ParamDecl((2,), "vector", "bias")}
+        if self.has_bias:
+            decls["up_bias"] = ParamDecl((self.intermediate_size,), "vector", "bias")
+            decls["down_bias"] = ParamDecl((self.hidden_size,), "vector", "bias")
+        return decls
+
+    up_weight = property(lambda s: s.up.weight, lambda s, t: setattr(s.up, "weight", t))
+    up_bias = property(lambda s: s.up.bias, lambda s, t: setattr(s.up, "bias", t))
+    down_weight = property(lambda s: s.down.weight, lambda s, t: setattr(s.down, "weight", t))
+
+    @property
+    def down_bias(self) -> Optional[torch.Tensor]:
+        return self.residual_bias if self.defer_bias else self.down.bias
+
+    @down_bias.setter
+    def down_bias(self, t) -> None:
+        if self.defer_bias:
+            self.residual_bias = t
+        else:
+            self.down.bias = t
+
+    def prepare(self, device, compute_dtype) -> None:
+        p, q = (float(v) for v in self.act.double().cpu())
+        self._act = ops.PointAct("xielu", _softplus(p), 0.5 + _softplus(q))
+        copies = bool(self.options.get("weight_copies", True))
+        self.up.prepare(copies)
+        self.down.prepare(copies)
+
+    def release_optional_memory(self) -> int:
+        return self.up.drop_copy() + self.down.drop_copy()
+
+    def _activated(self, x: torch.Tensor) -> torch.Tensor:
+        m, up = x.shape[0], self.up
+        if x.dtype == torch.bfloat16 and m > 0:
+            if up.streamed is not None and ops.gemm_mfma_wide_act_takes(m, up.streamed):
+                return ops.gemm_mfma_wide_act(x, up.streamed, up.bias, self._act)
+            if m <= GEMM_MFMA_SKINNY_BEST_M and self.hidden_size % 8 == 0:
+                return ops.gemm_mfma_skinny_act(x, up.weight, up.bias, self._act)
+            sums = up.partial_sums(x) if self.intermediate_size % 4 == 0 else None
+            if sums is not None:
+                return ops.sum_round(sums, up.bias, self._act)
+        y = up(x, skip_bias=True)
+        return ops.bias_act(y, up.bias, self._act, out=y)
+
+    def forward(self, x: torch.Tensor, ctx) -> torch.Tensor:
+        return self.down.for_residual(self._activated(x), ctx)

@@ -10,6 +10,11 @@ from .. import ops
 from .base import HiddenState, Norm, ParamDecl, register_part
 
 
+def _no_delta_bias(hidden: HiddenState, name: str) -> None:
+    if hidden.delta_bias is not None:
+        raise RuntimeError(f"{name}: the stream's pending delta comes with a bias, which is not added here")
+
+
 def _no_second_delta(hidden: HiddenState, name: str) -> None:
     if hidden.delta_scale != 1.0:
         raise RuntimeError(f"{name}: the stream's pending delta carries a factor of {hidden.delta_scale}, which this norm "
@@ -29,6 +34,7 @@ class RMSNorm(Norm):
     ``RMSNorm``), that norm, the sum and this norm are one kernel."""
 
     adds_partial_sums = True
+    adds_delta_bias = True
 
     graph_safe = True
 
@@ -50,11 +56,13 @@ class RMSNorm(Norm):
 
     def __call__(self, hidden: HiddenState, out_dtype: torch.dtype) -> torch.Tensor:
         _no_second_delta(hidden, "rms_norm")
-        delta, post = hidden.delta, hidden.delta_norm
-        hidden.delta = hidden.delta_norm = None
+        delta, post, bias = hidden.delta, hidden.delta_norm, hidden.delta_bias
+        if post is None:
+            _no_delta_bias(hidden, "rms_norm")
+        hidden.delta = hidden.delta_norm = hidden.delta_bias = None
         if delta is not None and post is not None:
             return ops.sandwich_norm(hidden.residual, delta, post.weight, post.eps, self.weight, self.eps, out_dtype,
-                                     write_back=True)
+                                     write_back=True, delta_bias=bias)
         return ops.rmsnorm(hidden.residual, self.weight, self.eps, out_dtype, delta=delta,
                            write_back=delta is not None)
 
@@ -63,7 +71,8 @@ class RMSNorm(Norm):
         if hidden.delta is not None and hidden.delta_norm is not None:
             post = hidden.delta_norm
             return ops.sandwich_norm(hidden.residual, hidden.delta, post.weight, post.eps, self.weight, self.eps,
-                                     out_dtype, rows=rows)
+                                     out_dtype, rows=rows, delta_bias=hidden.delta_bias)
+        _no_delta_bias(hidden, "rms_norm")
         return ops.rmsnorm(hidden.residual, self.weight, self.eps, out_dtype, delta=hidden.delta, rows=rows)
 
     def plain(self, x: torch.Tensor, out=None) -> torch.Tensor:
@@ -93,6 +102,7 @@ class LayerNorm(Norm):
 
     @staticmethod
     def _take(hidden: HiddenState, clear: bool):
+        _no_delta_bias(hidden, "layer_norm")
         if hidden.delta_norm is not None:
             raise RuntimeError("layer_norm: a pending delta with a norm of its own is not taken")
         if hidden.delta_scale != 1.0:
@@ -144,6 +154,7 @@ class GroupRMSNorm(Norm):
 
     @staticmethod
     def _take(hidden: HiddenState, clear: bool):
+        _no_delta_bias(hidden, "group_rms_norm")
         if hidden.delta_norm is not None:
             raise RuntimeError("group_rms_norm: a pending delta with a norm of its own is not taken")
         taken = hidden.delta, hidden.delta2, hidden.delta_scale
@@ -190,6 +201,7 @@ class StreamReader(Norm):
     @staticmethod
     def _pending(hidden: HiddenState):
         _no_second_delta(hidden, "stream")
+        _no_delta_bias(hidden, "stream")
         delta, post = hidden.delta, hidden.delta_norm
         if delta is not None and post is None:
             raise RuntimeError("stream: a pending delta without a norm of its own is not taken (a pre-norm block came before)")
