@@ -305,12 +305,29 @@ def mafosun_shape(width: int, ff: int, layers: int, vocab: int) -> dict:
     return {"architecture": "Mafosun", "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "layers": out}
 
 
-DESIGN_SHAPES = {"gilozen": gilozen_shape, "botulorn": botulorn_shape, "fiterax": fiterax_shape, "mafosun": mafosun_shape}
+def romepel_shape(width: int, ff: int, layers: int, vocab: int) -> dict:
+    """A Romepel configuration of real layer sizes: gated linear attention in every third layer, in the others
+    grouped-query attention over a window of 1,024 positions with a bias by distance and position-scaled queries, every
+    layer with a feed-forward of two matrices."""
+    heads = width // 128
+    gla = {"heads": heads // 2, "dim": 128, "vdim": 256, "tau": 16.0, "a_rank": 64}
+    gqa = {"heads": heads, "kv_heads": max(1, width // 512), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+           "mask": {"size": 1024}, "q_temp": {"coef": 0.2, "every": 512}}
+    out = [{"type": "gla" if i % 3 == 0 else "attention", "mixer": dict(gla if i % 3 == 0 else gqa),
+            "mlp": {"kind": "dense", "ff": ff}} for i in range(layers)]
+    return {"architecture": "Romepel", "width": width, "vocab": vocab, "max_positions": 8192, "norm": {"eps": 1e-5},
+            "logit_softcap": 30.0, "layers": out}
+
+
+DESIGN_SHAPES = {"gilozen": gilozen_shape, "botulorn": botulorn_shape, "fiterax": fiterax_shape, "mafosun": mafosun_shape,
+                 "romepel": romepel_shape}
+# a design whose mechanisms an earlier one shares is measured beside that one too
+DESIGN_BESIDE = {"romepel": ("gilozen",)}
 DESIGN_SIZES = {"2048": (2048, 8192, 9, 32000), "4096": (4096, 14336, 9, 32000)}  # width, ff, layers, vocab
 
 
 def design_comparison(args) -> int:
-    """--workload gilozen | botulorn | fiterax | mafosun: prefill (one prompt of 2,048 tokens in one step) and decode (batches of 8 and 64 at a
+    """--workload gilozen | botulorn | fiterax | mafosun | romepel: prefill (one prompt of 2,048 tokens in one step) and decode (batches of 8 and 64 at a
     context of 512, from captured graphs) of the named design at two real layer sizes with random weights, beside a Qwen2
     model of the same width, feed-forward, layers and vocabulary (grouped-query attention, 128 values a head, four
     query heads a key/value head) through the same step function.  One JSON line."""
@@ -330,7 +347,10 @@ def design_comparison(args) -> int:
                 "num_hidden_layers": layers, "num_attention_heads": width // 128, "num_key_value_heads": width // 512,
                 "head_dim": 128, "intermediate_size": ff, "vocab_size": vocab, "rope_theta": 500000.0,
                 "rms_norm_eps": 1e-5, "tie_word_embeddings": False, "max_position_embeddings": 8192}
-        for name, raw in ((args.workload, DESIGN_SHAPES[args.workload](width, ff, layers, vocab)), ("qwen2", qwen)):
+        designs = (args.workload, *DESIGN_BESIDE.get(args.workload, ()))
+        for name, raw in [(d, DESIGN_SHAPES[d](width, ff, layers, vocab)) for d in designs] + [("qwen2", qwen)]:
+            if args.design_models and name not in args.design_models.split(","):
+                continue
             model = Model.from_random(parse_config(raw), seed=0, dtype=dtype)
             pages_each = (512 + args.warmup + args.steps) // 16 + 2  # a decoding request's context and every step after it
             runner = Runner(model, page_size=16, num_pages=64 * max(40, pages_each) + 160, max_requests=64)
@@ -395,14 +415,15 @@ def main() -> int:
     ap.add_argument("--no-tune", action="store_true", help="leave the library's kernel choice for prefill to its heuristic")
     ap.add_argument("--no-streamed-copies", action="store_true",
                     help="do not keep the large weights a second time in the order of the matrix instruction's fragments")
-    ap.add_argument("--design-sizes", default="2048,4096", help="--workload gilozen | botulorn | fiterax | mafosun: widths to run (2048, 4096)")
-    ap.add_argument("--design-batches", default="8,64", help="--workload gilozen | botulorn | fiterax | mafosun: decode batches to time (at most 64)")
-    ap.add_argument("--design-phases", default="prefill,decode", help="--workload gilozen | botulorn | fiterax | mafosun: what to time (for a trace of one phase)")
-    ap.add_argument("--workload", choices=["decode", "mixed", "long-prefill", "gilozen", "botulorn", "fiterax", "mafosun"], default="decode",
+    ap.add_argument("--design-sizes", default="2048,4096", help="--workload gilozen | botulorn | fiterax | mafosun | romepel: widths to run (2048, 4096)")
+    ap.add_argument("--design-batches", default="8,64", help="--workload gilozen | botulorn | fiterax | mafosun | romepel: decode batches to time (at most 64)")
+    ap.add_argument("--design-phases", default="prefill,decode", help="--workload gilozen | botulorn | fiterax | mafosun | romepel: what to time (for a trace of one phase)")
+    ap.add_argument("--design-models", default="", help="--workload gilozen | botulorn | fiterax | mafosun | romepel: of the models compared, only these (for a trace of one)")
+    ap.add_argument("--workload", choices=["decode", "mixed", "long-prefill", "gilozen", "botulorn", "fiterax", "mafosun", "romepel"], default="decode",
                     help="decode: the default run.  mixed: --requests prompts of --min-prompt to --max-prompt tokens, "
                          "--outputs tokens each, through the scheduler (made for --shape 14b).  "
                          "long-prefill: one prompt of --prefill-tokens tokens in portions of the token budget "
-                         "(made for --shape 32b).  gilozen, botulorn, fiterax, mafosun: that design beside Qwen2 at equal layer sizes")
+                         "(made for --shape 32b).  gilozen, botulorn, fiterax, mafosun, romepel: that design beside Qwen2 at equal layer sizes")
     ap.add_argument("--requests", type=int, default=32)
     ap.add_argument("--min-prompt", type=int, default=128)
     ap.add_argument("--max-prompt", type=int, default=4096)

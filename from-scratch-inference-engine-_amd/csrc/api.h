@@ -202,12 +202,12 @@ int fsie_gemm_mfma_wide_gated(const void* x, const void* w, void* y, int M, int 
 // fragment-ordered weight)
 int fsie_gemm_mfma_wide_takes(int M, int N, int K, int splits, int gate_up, int frags);
 // y = act(x . w^T + bias) in bfloat16, act a FsiePointAct with its constants: by the few-rows product (up to 16 rows) and
-// by the one that shares x through LDS (its rows; one slice of K, N a multiple of 4)
+// by the one that shares x through LDS (up to 64 rows, one slice of K, N a multiple of 4)
 int fsie_gemm_mfma_skinny_act(const void* x, const void* w, const float* bias, void* y, int M, int N, int K, int waves,
                               int blocks, int act, float act_pos, float act_neg, hipStream_t stream);
 int fsie_gemm_mfma_wide_act(const void* x, const void* w, const float* bias, void* y, int M, int N, int K, int waves,
                             int blocks, int frags, int act, float act_pos, float act_neg, hipStream_t stream);
-int fsie_gemm_mfma_wide_act_takes(int M, int N, int K, int frags);
+int fsie_gemm_mfma_wide_act_takes(int M, int N, int K);
 int64_t fsie_fragment_order_size(int N, int K);
 int fsie_fragment_order(const void* w, void* out, int N, int K, hipStream_t stream);
 

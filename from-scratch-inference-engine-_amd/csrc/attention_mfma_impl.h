@@ -123,7 +123,9 @@ constexpr int max_waves() {
     return HDT <= 4 ? 16 : (HDT <= 8 ? 8 : 4);  // registers per wave grow with the head size
 }
 
-template <int HDT, int NT, int MAXW, bool V16, bool QKV = false>
+// BIASED false: no distance bias and no factor a token, known when the kernel is compiled (the QKV variants have no
+// registers to spare for them); true: whatever slopes and row_scale say.
+template <int HDT, int NT, int MAXW, bool V16, bool QKV = false, bool BIASED = true>
 __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((amdgpu_waves_per_eu(MAXW == 1 && NT > 1 ? 2 : 1))) void attention_mfma_kernel(
     const bf16_t* __restrict__ q, int64_t q_stride, const bf16_t* __restrict__ k_pool,
     const bf16_t* __restrict__ v_pool, const int32_t* __restrict__ block_tables, int max_pages,
@@ -180,7 +182,7 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
     const float cap2 = f.softcap * kLog2e, cap_in = capped ? scale / f.softcap : scale2;
     auto scaled = [&](float product, float in) { return capped ? cap2 * tanh_by_exp(product * in) : product * in; };
     // the distance bias, in the same units: slope (key - query), added to the scaled scores
-    const bool sloped = f.slopes != nullptr;
+    const bool sloped = BIASED && f.slopes != nullptr;
 
     // LDS: the accumulators that the waves after the first hand over at the end; before that, in
     // the QKV variant, the heads added up from the sums (up to 16 of queries, a key, a value) and
@@ -277,7 +279,7 @@ __global__ __launch_bounds__(QKV && MAXW == 1 ? 256 : 64 * MAXW) __attribute__((
         rtok[nt] = tq;
         rhead[nt] = h_base + hh;
         rpos[nt] = pos0 + tq;
-        r_in[nt] = f.row_scale ? cap_in * f.row_scale[q_row0 + (rvalid[nt] ? tq : 0)] : cap_in;
+        r_in[nt] = BIASED && f.row_scale ? cap_in * f.row_scale[q_row0 + (rvalid[nt] ? tq : 0)] : cap_in;
         r_slope[nt] = sloped ? f.slopes[rvalid[nt] ? rhead[nt] : h_base] * kLog2e : 0.f;
         if constexpr (!QKV) {
             const bf16_t* qp = q + static_cast<int64_t>(q_row0 + (rvalid[nt] ? tq : 0)) * q_stride +
@@ -771,13 +773,19 @@ int launch_qkv(const QkvSums& f, const void* k_pool, const void* v_pool, const i
     if (waves < 1) waves = 1;
     if (waves > MAXW) waves = MAXW;
 #define FSIE_ATTN_LAUNCH(W, THREADS)                                                                                 \
-    attention_mfma_kernel<HDT, 1, W, true, true><<<grid, THREADS, 0, stream>>>(                                      \
+    if (f.slopes || f.row_scale) FSIE_ATTN_LAUNCH_AS(W, THREADS, true); else FSIE_ATTN_LAUNCH_AS(W, THREADS, false)
+#define FSIE_ATTN_LAUNCH_AS(W, THREADS, B)                                                                           \
+    attention_mfma_kernel<HDT, 1, W, true, true, B><<<grid, THREADS, 0, stream>>>(                                      \
         nullptr, 0, static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool), block_tables, max_pages, \
         items, static_cast<bf16_t*>(out), partials, n_heads, n_kv, page_size, window, scale, gh, head_chunks, f)
     // one wave and three that only help with the sums; or all the waves the kernel has (those that an
     // item's keys leave idle help with the sums too)
-    if (waves == 1) FSIE_ATTN_LAUNCH(1, 256);
-    else FSIE_ATTN_LAUNCH(MAXW, 64 * MAXW);
+    if (waves == 1) {
+        FSIE_ATTN_LAUNCH(1, 256);
+    } else {
+        FSIE_ATTN_LAUNCH(MAXW, 64 * MAXW);
+    }
+#undef FSIE_ATTN_LAUNCH_AS
 #undef FSIE_ATTN_LAUNCH
     FSIE_CHECK_LAUNCH("attention_mfma_qkv");
     return 0;

@@ -327,16 +327,17 @@ __global__ __launch_bounds__(kLdsThreads) __attribute__((amdgpu_waves_per_eu(HDT
                                         (window <= 0 || kh > pos0 + n_q - 1 - window));
 #pragma unroll
             for (int nt = 0; nt < NT; ++nt) {
-                if constexpr (BIASED) {  // (the mask below then replaces the keys that a row does not see)
-                    const float at_first = r_slope[nt] * static_cast<float>(kh + 8 * G - rpos[nt]);
+                // the score of the i-th of this lane's eight keys
+                const float at_first = BIASED ? r_slope[nt] * static_cast<float>(kh + 8 * G - rpos[nt]) : 0.f;
+                auto score_at = [&](int i) {
+                    const float product = st[h][nt][i >> 2][i & 3];
+                    if constexpr (BIASED) return score_of(product * r_in[nt]) + fmaf(r_slope[nt], static_cast<float>(i), at_first);
+                    else return score_of(product);
+                };
+                if (full) {
 #pragma unroll
-                    for (int i = 0; i < 8; ++i)
-                        sv[h][nt][i] = score_of(st[h][nt][i >> 2][i & 3] * r_in[nt]) + fmaf(r_slope[nt], static_cast<float>(i), at_first);
+                    for (int i = 0; i < 8; ++i) sv[h][nt][i] = score_at(i);
                 } else {
-#pragma unroll
-                    for (int i = 0; i < 8; ++i) sv[h][nt][i] = score_of(st[h][nt][i >> 2][i & 3]);
-                }
-                if (!full) {
 #pragma unroll
                     for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
@@ -346,7 +347,7 @@ __global__ __launch_bounds__(kLdsThreads) __attribute__((amdgpu_waves_per_eu(HDT
                                                              : ((key >= key_begin && key < key_end) || key < kept_in_range);
                             const bool vis = rvalid[nt] && in_range && key <= rpos[nt] &&
                                              (window <= 0 || key > rpos[nt] - window || key < keep);
-                            sv[h][nt][tt * 4 + r] = vis ? sv[h][nt][tt * 4 + r] : -INFINITY;
+                            sv[h][nt][tt * 4 + r] = vis ? score_at(tt * 4 + r) : -INFINITY;
                         }
                 }
 #pragma unroll

@@ -68,10 +68,18 @@ __device__ __forceinline__ float gate_act(float g, int act) {
 // 1: xIELU, z / 2 plus pos * z^2 above zero and neg * (exp(z) - 1 - z) below it.
 enum FsiePointAct { FSIE_POINT_NONE = 0, FSIE_POINT_XIELU = 1 };
 #define FSIE_POINT_KNOWN(act) ((act) == FSIE_POINT_NONE || (act) == FSIE_POINT_XIELU)
+// exp(z) - 1 - z for z <= 0.  EXACT: within float32 roundings of z.  Else, for results that are rounded to 16 bits: the
+// series up to z^6 / 720 above -1/2 (its remainder there is below 2e-5 of the whole) and the hardware's exponential below.
+template <bool EXACT>
+__device__ __forceinline__ float exp_less_line(float z) {
+    if (EXACT) return expm1f(z) - z;
+    const float series = z * z * fmaf(z, fmaf(z, fmaf(z, fmaf(z, 1.f / 720.f, 1.f / 120.f), 1.f / 24.f), 1.f / 6.f), 0.5f);
+    return z > -0.5f ? series : __expf(z) - 1.f - z;
+}
+template <bool EXACT>
 __device__ __forceinline__ float point_act(float z, int act, float pos, float neg) {
     if (act == FSIE_POINT_NONE) return z;
-    const float below = fminf(z, 0.f);
-    return fmaf(0.5f, z, z > 0.f ? pos * z * z : neg * (expm1f(below) - below));
+    return fmaf(0.5f, z, z > 0.f ? pos * z * z : neg * exp_less_line<EXACT>(fminf(z, 0.f)));
 }
 
 // tanh through one exponential, 1 - 2 / (exp(2x) + 1): within a few float32 roundings of 1 in absolute terms,

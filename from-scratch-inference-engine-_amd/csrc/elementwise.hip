@@ -318,23 +318,34 @@ __global__ void bias_add_kernel(T* __restrict__ y, const float* __restrict__ bia
     if (i < total) y[i] = from_float<T>(to_float(y[i]) + bias[i % cols]);
 }
 
-// y = act(x + bias), one row a blockIdx.x; VEC: four values a thread
+// y = act(x + bias), one row a blockIdx.x; VEC: eight values a thread
 template <typename T, bool VEC>
 __global__ __launch_bounds__(kThreads) void bias_act_kernel(const T* __restrict__ x, const float* __restrict__ bias, T* __restrict__ y,
                                                             int cols, int act, float act_pos, float act_neg) {
-    const int j = (blockIdx.y * kThreads + threadIdx.x) * (VEC ? 4 : 1);
+    const int j = (blockIdx.y * kThreads + threadIdx.x) * (VEC ? 8 : 1);
     if (j >= cols) return;
     const int64_t i = static_cast<int64_t>(blockIdx.x) * cols + j;
     if constexpr (VEC) {
-        float4 v = Pack4<T>::load(x + i);
-        if (bias) {
-            const float4 b = Pack4<float>::load(bias + j);
-            v = float4{v.x + b.x, v.y + b.y, v.z + b.z, v.w + b.w};
+        constexpr bool EXACT = sizeof(T) == 4;
+        float4 v[2] = {Pack4<T>::load(x + i), Pack4<T>::load(x + i + 4)};
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            if (bias) {
+                const float4 b = Pack4<float>::load(bias + j + 4 * h);
+                v[h] = float4{v[h].x + b.x, v[h].y + b.y, v[h].z + b.z, v[h].w + b.w};
+            }
+            v[h] = float4{point_act<EXACT>(v[h].x, act, act_pos, act_neg), point_act<EXACT>(v[h].y, act, act_pos, act_neg),
+                          point_act<EXACT>(v[h].z, act, act_pos, act_neg), point_act<EXACT>(v[h].w, act, act_pos, act_neg)};
         }
-        Pack4<T>::store(y + i, float4{point_act(v.x, act, act_pos, act_neg), point_act(v.y, act, act_pos, act_neg),
-                                      point_act(v.z, act, act_pos, act_neg), point_act(v.w, act, act_pos, act_neg)});
+        if constexpr (EXACT) {
+            Pack4<T>::store(y + i, v[0]);
+            Pack4<T>::store(y + i + 4, v[1]);
+        } else {
+            *reinterpret_cast<uint4*>(y + i) = uint4{pack2_bf16(v[0].x, v[0].y), pack2_bf16(v[0].z, v[0].w),
+                                                     pack2_bf16(v[1].x, v[1].y), pack2_bf16(v[1].z, v[1].w)};
+        }
     } else {
-        y[i] = from_float<T>(point_act(to_float(x[i]) + (bias ? bias[j] : 0.f), act, act_pos, act_neg));
+        y[i] = from_float<T>(point_act<sizeof(T) == 4>(to_float(x[i]) + (bias ? bias[j] : 0.f), act, act_pos, act_neg));
     }
 }
 
@@ -361,8 +372,8 @@ __global__ void sum_round_kernel(const float* __restrict__ parts, int planes, in
         sum.x += b.x, sum.y += b.y, sum.z += b.z, sum.w += b.w;
     }
     if (act != FSIE_POINT_NONE)
-        sum = float4{point_act(sum.x, act, act_pos, act_neg), point_act(sum.y, act, act_pos, act_neg),
-                     point_act(sum.z, act, act_pos, act_neg), point_act(sum.w, act, act_pos, act_neg)};
+        sum = float4{point_act<false>(sum.x, act, act_pos, act_neg), point_act<false>(sum.y, act, act_pos, act_neg),
+                     point_act<false>(sum.z, act, act_pos, act_neg), point_act<false>(sum.w, act, act_pos, act_neg)};
     uint2 raw;
     raw.x = static_cast<uint32_t>(from_float<bf16_t>(sum.x).bits) | static_cast<uint32_t>(from_float<bf16_t>(sum.y).bits) << 16;
     raw.y = static_cast<uint32_t>(from_float<bf16_t>(sum.z).bits) | static_cast<uint32_t>(from_float<bf16_t>(sum.w).bits) << 16;
@@ -658,9 +669,9 @@ extern "C" int fsie_bias_act(const void* x, const float* bias, void* y, int rows
     FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "bias_act: unknown dtype %d", dtype);
     FSIE_REQUIRE(FSIE_POINT_KNOWN(act), "bias_act: unknown activation %d", act);
     if (rows == 0) return 0;
-    const bool vec = cols % 4 == 0 && ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(y) |
+    const bool vec = cols % 8 == 0 && ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(y) |
                                         reinterpret_cast<uintptr_t>(bias)) & 15) == 0;
-    const dim3 grid(static_cast<unsigned>(rows), static_cast<unsigned>(ceil_div64(vec ? cols / 4 : cols, kThreads)));
+    const dim3 grid(static_cast<unsigned>(rows), static_cast<unsigned>(ceil_div64(vec ? cols / 8 : cols, kThreads)));
 #define FSIE_BIAS_ACT(T, V) \
     bias_act_kernel<T, V><<<grid, kThreads, 0, stream>>>(static_cast<const T*>(x), bias, static_cast<T*>(y), cols, act, act_pos, act_neg)
     if (dtype == FSIE_F32) {

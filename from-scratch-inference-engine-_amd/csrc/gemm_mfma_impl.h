@@ -292,7 +292,7 @@ __global__ __launch_bounds__(WAVES * FSIE_WAVE) void gemm_mfma_skinny_kernel(
                 const int nn = n0 + nb * 16 + kg * 4 + r;
                 if (nn < N) {
                     float v = bias ? acc[nb][t][r] + bias[nn] : acc[nb][t][r];
-                    if constexpr (EPI == EPI_PLAIN && sizeof(OutT) == 2) v = point_act(v, act, act_pos, act_neg);
+                    if constexpr (EPI == EPI_PLAIN && sizeof(OutT) == 2) v = point_act<false>(v, act, act_pos, act_neg);
                     y[static_cast<int64_t>(m) * N + nn] = from_float<OutT>(v);
                 }
             }

@@ -55,9 +55,11 @@ union Frag {
     bf16x8 v;
 };
 
-// What becomes of a sum where the result is not float32: y bfloat16 [M, N] = act(sum + bias), act a FsiePointAct.
+// What becomes of the sums: SUMS float32, GATED bfloat16 [M, N / 2] from gate and up rows in turn, POINT bfloat16 [M, N] =
+// act(sum + bias), act a FsiePointAct.
+enum Result { SUMS, GATED, POINT };
 struct PointEpilogue {
-    int act = FSIE_POINT_NONE;  // NONE: float32 sums without bias
+    int act = FSIE_POINT_NONE;
     float pos = 0.f, neg = 0.f;
     const float* bias = nullptr;
 };
@@ -65,9 +67,9 @@ struct PointEpilogue {
 // MT tiles of 16 rows of X; WAVES waves of NB blocks of 16 rows of W each per workgroup (a wave's
 // blocks share the B fragments it reads from LDS: with four tiles of X one block a wave would be
 // bound by those reads); STEPS 32-wide MFMA steps per stage (KS = 32 * STEPS values of K).
-// SWIGLU: the rows of W are gate and up interleaved and y is bfloat16 [M, N / 2], silu(gate) * up
+// GATED: the rows of W are gate and up interleaved and y is bfloat16 [M, N / 2], silu(gate) * up
 // from the accumulators (a lane holds rows 4 kg .. 4 kg + 3 of a block: two pairs); one slice only.
-template <int MT, int WAVES, int STEPS, int NB, bool SWIGLU, bool FRAGS>
+template <int MT, int WAVES, int STEPS, int NB, int RESULT, bool FRAGS>
 __global__ __launch_bounds__(WAVES * 64) void gemm_mfma_wide_kernel(const bf16_t* __restrict__ x,
                                                                    const bf16_t* __restrict__ w,
                                                                    float* __restrict__ y, int M, int N, int K,
@@ -190,7 +192,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_mfma_wide_kernel(const bf16_t
     }
 
     // lane holds D[n0 + 16 nb + 4 kg + r][m = 16 t + row]
-    if constexpr (SWIGLU) {
+    if constexpr (RESULT == GATED) {
         uint32_t* out = reinterpret_cast<uint32_t*>(y);  // two bfloat16 results a store: columns nn / 2 and nn / 2 + 1
 #pragma unroll
         for (int nb = 0; nb < NB; ++nb)
@@ -205,7 +207,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_mfma_wide_kernel(const bf16_t
             }
         return;
     }
-    if (point.act != FSIE_POINT_NONE) {
+    if constexpr (RESULT == POINT) {
         uint2* out = reinterpret_cast<uint2*>(y);
 #pragma unroll
         for (int nb = 0; nb < NB; ++nb)
@@ -217,7 +219,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_mfma_wide_kernel(const bf16_t
                 float v[4];
 #pragma unroll
                 for (int r = 0; r < 4; ++r)
-                    v[r] = point_act(acc[nb][t][r] + (point.bias ? point.bias[nn + r] : 0.f), point.act, point.pos, point.neg);
+                    v[r] = point_act<false>(acc[nb][t][r] + (point.bias ? point.bias[nn + r] : 0.f), point.act, point.pos, point.neg);
                 out[(static_cast<int64_t>(m) * N + nn) / 4] = uint2{pack2_bf16(v[0], v[1]), pack2_bf16(v[2], v[3])};
             }
         return;
@@ -237,7 +239,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_mfma_wide_kernel(const bf16_t
         }
 }
 
-template <int MT, int WAVES, int STEPS, int NB, bool SWIGLU, bool FRAGS>
+template <int MT, int WAVES, int STEPS, int NB, int RESULT, bool FRAGS>
 int launch(const bf16_t* x, const bf16_t* w, float* y, int M, int N, int K, int splits, int k_slice,
            int act, const PointEpilogue& point, hipStream_t stream) {
     const int rows = 16 * NB * WAVES;
@@ -246,35 +248,35 @@ int launch(const bf16_t* x, const bf16_t* w, float* y, int M, int N, int K, int 
     constexpr int dynamic = lds > kStaticLds ? lds : 0;
     if constexpr (dynamic > 0) {
         static const hipError_t allowed = hipFuncSetAttribute(
-            reinterpret_cast<const void*>(&gemm_mfma_wide_kernel<MT, WAVES, STEPS, NB, SWIGLU, FRAGS>),
+            reinterpret_cast<const void*>(&gemm_mfma_wide_kernel<MT, WAVES, STEPS, NB, RESULT, FRAGS>),
             hipFuncAttributeMaxDynamicSharedMemorySize, dynamic);
         if (allowed != hipSuccess) {
             fsie_set_error("gemm_mfma_wide: %d bytes of LDS for %d rows: %s", dynamic, M, hipGetErrorString(allowed));
             return 1;
         }
     }
-    gemm_mfma_wide_kernel<MT, WAVES, STEPS, NB, SWIGLU, FRAGS><<<grid, WAVES * 64, dynamic, stream>>>(x, w, y, M, N, K, k_slice, act, point);
+    gemm_mfma_wide_kernel<MT, WAVES, STEPS, NB, RESULT, FRAGS><<<grid, WAVES * 64, dynamic, stream>>>(x, w, y, M, N, K, k_slice, act, point);
     FSIE_CHECK_LAUNCH("gemm_mfma_wide");
     return 0;
 }
 
-template <int WAVES, int STEPS, int NB, bool SWIGLU, bool FRAGS>
+template <int WAVES, int STEPS, int NB, int RESULT, bool FRAGS>
 int launch_mt(int mt, const bf16_t* x, const bf16_t* w, float* y, int M, int N, int K, int splits, int k_slice, int act,
               const PointEpilogue& point, hipStream_t stream) {
     switch (mt) {
-        case 1: return launch<1, WAVES, STEPS, NB, SWIGLU, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
-        case 2: return launch<2, WAVES, STEPS, NB, SWIGLU, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        case 1: return launch<1, WAVES, STEPS, NB, RESULT, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        case 2: return launch<2, WAVES, STEPS, NB, RESULT, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
 #if FSIE_WIDE_STEPS <= 4
-        case 3: return launch<3, WAVES, STEPS, NB, SWIGLU, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
-        case 4: return launch<4, WAVES, STEPS, NB, SWIGLU, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        case 3: return launch<3, WAVES, STEPS, NB, RESULT, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        case 4: return launch<4, WAVES, STEPS, NB, RESULT, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
         default:
             // five to eight tiles of X (65 to 128 rows): on a fragment-ordered weight, two row blocks a
             // wave, four waves and more
-            if constexpr (FRAGS && NB == 2 && WAVES >= 4) {
-                if (mt == 8) return launch<8, WAVES, STEPS, NB, SWIGLU, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
-                if (mt == 5) return launch<5, WAVES, STEPS, NB, SWIGLU, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
-                if (mt == 6) return launch<6, WAVES, STEPS, NB, SWIGLU, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
-                if (mt == 7) return launch<7, WAVES, STEPS, NB, SWIGLU, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
+            if constexpr (FRAGS && NB == 2 && WAVES >= 4 && RESULT != POINT) {
+                if (mt == 8) return launch<8, WAVES, STEPS, NB, RESULT, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
+                if (mt == 5) return launch<5, WAVES, STEPS, NB, RESULT, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
+                if (mt == 6) return launch<6, WAVES, STEPS, NB, RESULT, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
+                if (mt == 7) return launch<7, WAVES, STEPS, NB, RESULT, FRAGS>(x, w, y, M, N, K, splits, k_slice, act, point, stream);
             }
             fsie_set_error("gemm_mfma_wide: %d rows only on a fragment-ordered weight with two row blocks a wave and "
                            "at least four waves (N = %d in %d slices gives %d blocks, %d waves)", M, N, splits, NB, WAVES);
@@ -285,23 +287,23 @@ int launch_mt(int mt, const bf16_t* x, const bf16_t* w, float* y, int M, int N, 
     }
 }
 
-template <bool SWIGLU, bool FRAGS>
+template <int RESULT, bool FRAGS>
 int launch_shape_of(int mt, int waves, int blocks, const bf16_t* x, const bf16_t* w, float* y, int M, int N, int K,
                     int splits, int k_slice, int act, const PointEpilogue& point, hipStream_t stream) {
-    if constexpr (SWIGLU && FRAGS) {  // gate/up of 17 rows and more: any number of waves that deals the rows evenly
-        if (blocks == 2 && waves == 3) return launch_mt<3, FSIE_WIDE_STEPS, 2, true, true>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
-        if (blocks == 2 && waves == 5) return launch_mt<5, FSIE_WIDE_STEPS, 2, true, true>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
-        if (blocks == 2 && waves == 6) return launch_mt<6, FSIE_WIDE_STEPS, 2, true, true>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
-        if (blocks == 2 && waves == 7) return launch_mt<7, FSIE_WIDE_STEPS, 2, true, true>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+    if constexpr (RESULT == GATED && FRAGS) {  // gate/up of 17 rows and more: any number of waves that deals the rows evenly
+        if (blocks == 2 && waves == 3) return launch_mt<3, FSIE_WIDE_STEPS, 2, GATED, true>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        if (blocks == 2 && waves == 5) return launch_mt<5, FSIE_WIDE_STEPS, 2, GATED, true>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        if (blocks == 2 && waves == 6) return launch_mt<6, FSIE_WIDE_STEPS, 2, GATED, true>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        if (blocks == 2 && waves == 7) return launch_mt<7, FSIE_WIDE_STEPS, 2, GATED, true>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
     }
     if (blocks == 2) {
-        if (waves == 8) return launch_mt<8, FSIE_WIDE_STEPS, 2, SWIGLU, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
-        if (waves == 2) return launch_mt<2, FSIE_WIDE_STEPS, 2, SWIGLU, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
-        return launch_mt<4, FSIE_WIDE_STEPS, 2, SWIGLU, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        if (waves == 8) return launch_mt<8, FSIE_WIDE_STEPS, 2, RESULT, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        if (waves == 2) return launch_mt<2, FSIE_WIDE_STEPS, 2, RESULT, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+        return launch_mt<4, FSIE_WIDE_STEPS, 2, RESULT, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
     }
-    if (waves == 8) return launch_mt<8, FSIE_WIDE_STEPS, 1, SWIGLU, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
-    if (waves == 2) return launch_mt<2, FSIE_WIDE_STEPS, 1, SWIGLU, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
-    return launch_mt<4, FSIE_WIDE_STEPS, 1, SWIGLU, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+    if (waves == 8) return launch_mt<8, FSIE_WIDE_STEPS, 1, RESULT, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+    if (waves == 2) return launch_mt<2, FSIE_WIDE_STEPS, 1, RESULT, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
+    return launch_mt<4, FSIE_WIDE_STEPS, 1, RESULT, FRAGS>(mt, x, w, y, M, N, K, splits, k_slice, act, point, stream);
 }
 
 // One thread a 16-byte unit of the copy: unit ((block, step), lane) holds the 8 values at row
@@ -467,8 +469,8 @@ extern "C" int fsie_gemm_mfma_wide(const void* x, const void* w, float* y, int M
     launch_shape(mt, N, splits, waves, blocks, false, frags != 0);
     const bf16_t* xp = static_cast<const bf16_t*>(x);
     const bf16_t* wq = static_cast<const bf16_t*>(w);
-    if (frags) return launch_shape_of<false, true>(mt, waves, blocks, xp, wq, y, M, N, K, splits, k_slice, 0, PointEpilogue{}, stream);
-    return launch_shape_of<false, false>(mt, waves, blocks, xp, wq, y, M, N, K, splits, k_slice, 0, PointEpilogue{}, stream);
+    if (frags) return launch_shape_of<SUMS, true>(mt, waves, blocks, xp, wq, y, M, N, K, splits, k_slice, 0, PointEpilogue{}, stream);
+    return launch_shape_of<SUMS, false>(mt, waves, blocks, xp, wq, y, M, N, K, splits, k_slice, 0, PointEpilogue{}, stream);
 }
 
 // The same product with the rows of w as gate and up in turn: y is bfloat16 [M, N / 2], silu(gate) * up.
@@ -496,8 +498,8 @@ extern "C" int fsie_gemm_mfma_wide_gated(const void* x, const void* w, void* y, 
     const bf16_t* xp = static_cast<const bf16_t*>(x);
     const bf16_t* wq = static_cast<const bf16_t*>(w);
     float* yp = static_cast<float*>(y);
-    if (frags) return launch_shape_of<true, true>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, act, PointEpilogue{}, stream);
-    return launch_shape_of<true, false>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, act, PointEpilogue{}, stream);
+    if (frags) return launch_shape_of<GATED, true>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, act, PointEpilogue{}, stream);
+    return launch_shape_of<GATED, false>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, act, PointEpilogue{}, stream);
 }
 
 // y = act(x . w^T + bias) in bfloat16 [M, N], act a FsiePointAct: one slice of K, N a multiple of 4.
@@ -506,7 +508,7 @@ extern "C" int fsie_gemm_mfma_wide_act(const void* x, const void* w, const float
                                        hipStream_t stream) {
     FSIE_REQUIRE(FSIE_POINT_KNOWN(act) && act != FSIE_POINT_NONE, "gemm_mfma_wide_act: unknown activation %d", act);
     FSIE_REQUIRE(M >= 0 && N > 0 && K > 0 && N % 4 == 0, "gemm_mfma_wide_act: bad sizes M=%d N=%d K=%d (N a multiple of 4)", M, N, K);
-    FSIE_REQUIRE(M <= (frags ? FSIE_GEMM_MFMA_WIDE_MAX_M : FSIE_GEMM_MFMA_SKINNY_MAX_M), "gemm_mfma_wide_act: too many rows, %d", M);
+    FSIE_REQUIRE(M <= FSIE_GEMM_MFMA_SKINNY_MAX_M, "gemm_mfma_wide_act: at most %d rows, got %d", FSIE_GEMM_MFMA_SKINNY_MAX_M, M);
     const int k_slice = fsie_gemm_mfma_wide_slice(K, 1);
     FSIE_REQUIRE(k_slice > 0, "gemm_mfma_wide_act: K=%d must be a multiple of the stage of %d", K, 32 * FSIE_WIDE_STEPS);
     FSIE_REQUIRE(reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0 &&
@@ -516,23 +518,22 @@ extern "C" int fsie_gemm_mfma_wide_act(const void* x, const void* w, const float
     FSIE_REQUIRE(blocks == 0 || blocks == 1 || blocks == 2, "gemm_mfma_wide_act: blocks must be 0, 1 or 2");
     if (M == 0) return 0;
     const int mt = (M + 15) / 16;
-    launch_shape(mt, N, 1, waves, blocks, true, false);  // (the waves that exist for both orders of w)
+    // Two waves a workgroup; one tile of x: two blocks of w a wave, more: one (MI355X, fragment-ordered, N = 8192, K = 2048:
+    // 8 rows 10.9 us against 12.3 with one block and 13.2 with four waves, 32 rows 11.2 against 13.8 and 14.8, 64 rows 16.0
+    // against 20.0 and 18.3; N = 14336, K = 4096: 8 rows 23.2 / 23.9 / 26.4, 32 rows 24.4 / 25.8 / 28.2)
+    if (waves == 0) waves = 2;
+    if (blocks == 0) blocks = mt == 1 ? 2 : 1;
     const PointEpilogue point{act, act_pos, act_neg, bias};
     const bf16_t* xp = static_cast<const bf16_t*>(x);
     const bf16_t* wq = static_cast<const bf16_t*>(w);
     float* yp = static_cast<float*>(y);
-    if (frags) return launch_shape_of<false, true>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, 0, point, stream);
-    return launch_shape_of<false, false>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, 0, point, stream);
+    if (frags) return launch_shape_of<POINT, true>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, 0, point, stream);
+    return launch_shape_of<POINT, false>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, 0, point, stream);
 }
 
 // Whether fsie_gemm_mfma_wide_act takes M rows of this shape.
-extern "C" int fsie_gemm_mfma_wide_act_takes(int M, int N, int K, int frags) {
-    if (M <= 0 || N <= 0 || N % 4 || fsie_gemm_mfma_wide_slice(K, 1) <= 0) return 0;
-    if (M <= FSIE_GEMM_MFMA_SKINNY_MAX_M) return 1;
-    if (!frags || M > FSIE_GEMM_MFMA_WIDE_MAX_M || FSIE_WIDE_STEPS > 4) return 0;
-    int waves = 0, blocks = 0;
-    launch_shape((M + 15) / 16, N, 1, waves, blocks, true, false);
-    return blocks == 2 && waves >= 4;
+extern "C" int fsie_gemm_mfma_wide_act_takes(int M, int N, int K) {
+    return M > 0 && M <= FSIE_GEMM_MFMA_SKINNY_MAX_M && N > 0 && N % 4 == 0 && fsie_gemm_mfma_wide_slice(K, 1) > 0;
 }
 
 extern "C" int fsie_gemm_mfma_wide_swiglu(const void* x, const void* w, void* y, int M, int N, int K, int waves,

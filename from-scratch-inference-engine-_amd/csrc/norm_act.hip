@@ -73,7 +73,7 @@ __device__ __forceinline__ void store4(bf16_t* p, float4 v) {
 // The same for hidden % 4 == 0 and hidden <= 4 * THREADS * ITERS: a thread keeps its quads of the row in
 // registers, and every load of the row (stream, delta or partial sums, both weights) goes out before
 // anything waits.  Places past the end read the last quad again and are masked out of sums and stores.
-template <typename T, int ITERS, int THREADS>
+template <typename T, int ITERS, int THREADS, bool BIAS>
 __global__ __launch_bounds__(THREADS) void sandwich_norm_vec_kernel(
     float* __restrict__ residual, const T* __restrict__ delta, const float* __restrict__ delta_bias,
     const float* __restrict__ post_weight, float post_eps,
@@ -92,6 +92,8 @@ __global__ __launch_bounds__(THREADS) void sandwich_norm_vec_kernel(
         v[it] = load4(res + j);
         wp[it] = load4(post_weight + j);
         w[it] = weight ? load4(weight + j) : float4{1.f, 1.f, 1.f, 1.f};
+        float4 b;
+        if (BIAS) b = load4(delta_bias + j);
         if (del) {
             y[it] = load4(del + j);
         } else {
@@ -103,10 +105,7 @@ __global__ __launch_bounds__(THREADS) void sandwich_norm_vec_kernel(
             }
             y[it] = a;
         }
-        if (delta_bias) {
-            const float4 b = load4(delta_bias + j);
-            y[it].x += b.x, y[it].y += b.y, y[it].z += b.z, y[it].w += b.w;
-        }
+        if (BIAS) y[it].x += b.x, y[it].y += b.y, y[it].z += b.z, y[it].w += b.w;
     }
     float sum_sq = 0.f;
 #pragma unroll
@@ -203,16 +202,18 @@ extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const floa
                          reinterpret_cast<uintptr_t>(weight) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
     if (aligned && hidden <= 8192) {
 #define FSIE_SANDWICH(T, ITERS, THREADS)                                                                             \
-    sandwich_norm_vec_kernel<T, ITERS, THREADS><<<n_rows, THREADS, 0, stream>>>(                                     \
+    if (delta_bias) FSIE_SANDWICH_WITH(T, ITERS, THREADS, true); else FSIE_SANDWICH_WITH(T, ITERS, THREADS, false)
+#define FSIE_SANDWICH_WITH(T, ITERS, THREADS, BIAS)                                                                  \
+    sandwich_norm_vec_kernel<T, ITERS, THREADS, BIAS><<<n_rows, THREADS, 0, stream>>>(                                     \
         residual, static_cast<const T*>(delta), delta_bias, post_weight, post_eps, weight, eps, static_cast<T*>(out), rows, hidden, \
         write_back, n_parts, part_stride)
 #define FSIE_SANDWICH_BY_SIZE(T)                                                      \
     if (n_rows <= 128 && hidden > 1024) {  /* few rows: more waves a row */           \
-        if (hidden <= 4096) FSIE_SANDWICH(T, 1, 1024); else FSIE_SANDWICH(T, 2, 1024); \
-    } else if (hidden <= 1024) FSIE_SANDWICH(T, 1, 256);                              \
-    else if (hidden <= 2048) FSIE_SANDWICH(T, 2, 256);                                \
-    else if (hidden <= 4096) FSIE_SANDWICH(T, 4, 256);                                \
-    else FSIE_SANDWICH(T, 8, 256)
+        if (hidden <= 4096) { FSIE_SANDWICH(T, 1, 1024); } else { FSIE_SANDWICH(T, 2, 1024); } \
+    } else if (hidden <= 1024) { FSIE_SANDWICH(T, 1, 256);                            \
+    } else if (hidden <= 2048) { FSIE_SANDWICH(T, 2, 256);                            \
+    } else if (hidden <= 4096) { FSIE_SANDWICH(T, 4, 256);                            \
+    } else { FSIE_SANDWICH(T, 8, 256); }
         if (dtype == FSIE_F32) {
             FSIE_SANDWICH_BY_SIZE(float);
         } else {
@@ -220,6 +221,7 @@ extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const floa
         }
 #undef FSIE_SANDWICH_BY_SIZE
 #undef FSIE_SANDWICH
+#undef FSIE_SANDWICH_WITH
         FSIE_CHECK_LAUNCH("sandwich_norm");
         return 0;
     }

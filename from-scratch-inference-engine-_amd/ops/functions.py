@@ -518,7 +518,7 @@ def gemm_mfma_wide_swiglu(x: torch.Tensor, weight: torch.Tensor, waves: int = 0,
 def gemm_mfma_wide_act(x: torch.Tensor, weight, bias: Optional[torch.Tensor], act: PointAct, waves: int = 0,
                        blocks: int = 0) -> torch.Tensor:
     """act(x . weight^T + bias) [M, N] in bfloat16 by the kernel that shares x through LDS, the activation in its epilogue
-    (``weight`` or its ``FragmentOrdered`` copy): N a multiple of 4, K of 128, rows as ``gemm_mfma_wide_act_takes`` says."""
+    (``weight`` or its ``FragmentOrdered`` copy): up to 64 rows, N a multiple of 4, K of 128."""
     _need(x, "gemm x", dtype=torch.bfloat16, ndim=2)
     m, k = x.shape
     wptr, n, frags = _wide_weight(weight, k)
@@ -533,7 +533,7 @@ def gemm_mfma_wide_act(x: torch.Tensor, weight, bias: Optional[torch.Tensor], ac
 def gemm_mfma_wide_act_takes(m: int, weight) -> bool:
     """Whether ``gemm_mfma_wide_act`` takes ``m`` rows against this weight."""
     n, k = weight.shape
-    return bool(load().fsie_gemm_mfma_wide_act_takes(int(m), int(n), int(k), int(isinstance(weight, FragmentOrdered))))
+    return bool(load().fsie_gemm_mfma_wide_act_takes(int(m), int(n), int(k)))
 
 
 def gemm_mfma_wide_best_splits(m: int, n: int, k: int) -> int:

@@ -57,7 +57,7 @@ _SIGNATURES = {
     "fsie_gemm_mfma_wide_swiglu": ([_P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_gemm_mfma_skinny_act": ([_P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, _P], c_int),
     "fsie_gemm_mfma_wide_act": ([_P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, _P], c_int),
-    "fsie_gemm_mfma_wide_act_takes": ([c_int, c_int, c_int, c_int], c_int),
+    "fsie_gemm_mfma_wide_act_takes": ([c_int, c_int, c_int], c_int),
     "fsie_gemm_mfma_wide_takes": ([c_int, c_int, c_int, c_int, c_int, c_int], c_int),
     "fsie_fragment_order_size": ([c_int, c_int], c_int64),
     "fsie_fragment_order": ([_P, _P, c_int, c_int, _P], c_int),

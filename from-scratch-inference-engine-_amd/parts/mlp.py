@@ -149,7 +149,10 @@ class PlainFeedForward(FeedForward):
     def _activated(self, x: torch.Tensor) -> torch.Tensor:
         m, up = x.shape[0], self.up
         if x.dtype == torch.bfloat16 and m > 0:
-            if up.streamed is not None and ops.gemm_mfma_wide_act_takes(m, up.streamed):
+            if (up.streamed is not None and ops.gemm_mfma_wide_act_takes(m, up.streamed)
+                    and (m <= 48 or self.intermediate_size <= 32 * ops.compute_units())):
+                # (a full fourth tile of x keeps a unit busy by itself: with more than a workgroup a unit the product in
+                # slices of K, 64 rows of N = 14336, K = 4096 30.7 us against 34.1)
                 return ops.gemm_mfma_wide_act(x, up.streamed, up.bias, self._act)
             if m <= GEMM_MFMA_SKINNY_BEST_M and self.hidden_size % 8 == 0:
                 return ops.gemm_mfma_skinny_act(x, up.weight, up.bias, self._act)
