@@ -65,8 +65,10 @@ int fsie_zero_pages(void* pool_a, void* pool_b, const int32_t* pages, int n, int
 // Counter-based random values (the random-weights mode): see elementwise.hip.
 int fsie_random_fill(void* out, int64_t n, uint64_t key, int kind, float std, hipStream_t stream);
 int fsie_swiglu(const void* x, void* out, int n_tokens, int inter, int dtype, hipStream_t stream);
-// the same with the gate's activation named: 0 = SiLU, 1 = GELU in its tanh form
-int fsie_gated_act(const void* x, void* out, int n_tokens, int inter, int dtype, int act, hipStream_t stream);
+// the same with the gate's activation named: 0 = SiLU, 1 = GELU in its tanh form, 2 = max(gate, 0); 3 = gate and up value
+// cut off at limit, g sigmoid(slope g) (u + 1) (limit and slope are read for that one only)
+int fsie_gated_act(const void* x, void* out, int n_tokens, int inter, int dtype, int act, float limit, float slope,
+                   hipStream_t stream);
 // The norm of a sublayer's output, the residual sum and the next norm in one pass:
 //   v = residual + rmsnorm(delta; post_weight, post_eps);  out = rmsnorm(v; weight, eps)
 // delta as for fsie_rmsnorm (one array of the activations' type, or n_parts float32 partial sums), plus delta_bias
@@ -74,6 +76,11 @@ int fsie_gated_act(const void* x, void* out, int n_tokens, int inter, int dtype,
 int fsie_sandwich_norm(float* residual, const void* delta, const float* delta_bias, const float* post_weight,
                        float post_eps, const float* weight, float eps, void* out, const int32_t* rows, int n_rows,
                        int hidden, int dtype, int write_back, int n_parts, int total_rows, hipStream_t stream);
+// out[row][0 .. hidden) = residual[row] + what is pending (nothing, delta itself, or with post_weight its RMS norm), rounded
+// to `dtype`, rows out_stride values apart; then residual[row] = restart (float32 [hidden]).  delta as for fsie_rmsnorm.
+int fsie_stream_out(float* residual, const void* delta, const float* post_weight, float post_eps, void* out,
+                    int64_t out_stride, const float* restart, int n_rows, int hidden, int dtype, int n_parts,
+                    hipStream_t stream);
 // out[t][h][:] = rmsnorm(o[t][h][:]; weight, eps) * act(gate[t][h][:]), a head `width` values wide; o float32, the sum
 // in order of n_planes arrays [n_tokens][heads * width] that lie one after the other
 int fsie_gated_headnorm(const float* o, int n_planes, const void* gate, int64_t gate_stride, const float* weight, void* out,
@@ -107,9 +114,13 @@ int fsie_rope_pairs(const void* in, int64_t in_stride, int in_off, int in_hs, vo
                     int out_hs, int heads, int width, int rot_pairs, int out_width, const float* cos_sin, int n_tokens,
                     int dtype, hipStream_t stream);
 int fsie_head_gemm(const void* x, int64_t x_stride, int x_off, int x_hs, const void* w, void* y, int64_t y_stride, int y_off,
-                   int y_hs, const float* gate, int n_tokens, int heads, int N, int K, int dtype, hipStream_t stream);
+                   int y_hs, const float* gate, const void* gate_rows, int64_t gate_stride, int rot_in, int rot_out,
+                   int rot_width, int rot_pairs, int rot_out_width, const float* cos_sin, int n_tokens, int heads, int N, int K,
+                   int dtype, hipStream_t stream);
 // y = x rounded to `dtype` (a copy for float32)
 int fsie_round_to(const float* x, void* y, int64_t total, int dtype, hipStream_t stream);
+// the same into columns of wider rows: y[r][0 .. cols), rows y_stride values apart
+int fsie_round_columns(const float* x, void* y, int64_t y_stride, int rows, int cols, int dtype, hipStream_t stream);
 // y = a * x1 + b * x2, elementwise, float32 arithmetic, all three of `dtype`
 int fsie_scaled_sum(const void* x1, float a, const void* x2, float b, void* y, int64_t total, int dtype, hipStream_t stream);
 int fsie_residual_add(float* residual, const void* delta, int64_t total, int dtype, hipStream_t stream);
@@ -192,9 +203,11 @@ int fsie_gemm_mfma_wide(const void* x, const void* w, float* y, int M, int N, in
 // the rows of w are gate and up in turn: y is bfloat16 [M, N / 2], silu(gate) * up
 int fsie_gemm_mfma_wide_swiglu(const void* x, const void* w, void* y, int M, int N, int K, int waves, int blocks,
                                int frags, hipStream_t stream);
-// the same with the gate's activation named (0 = SiLU, 1 = GELU in its tanh form)
+// the same with the gate's activation named (as for fsie_gated_act), here and by the few-rows product (up to 16 rows)
 int fsie_gemm_mfma_wide_gated(const void* x, const void* w, void* y, int M, int N, int K, int waves, int blocks,
-                              int frags, int act, hipStream_t stream);
+                              int frags, int act, float limit, float slope, hipStream_t stream);
+int fsie_gemm_mfma_skinny_gated(const void* x, const void* w, void* y, int M, int N, int K, int waves, int blocks, int act,
+                                float limit, float slope, hipStream_t stream);
 // A bfloat16 matrix [N, K] (K a multiple of 32) copied so that the 64 16-byte units of a block of 16
 // rows and 32 values of K lie together in the order of the lanes that hold them: a wave's load of W
 // is then one piece of 1 KB.  The copy has fsie_fragment_order_size values (N rounded up to 16 rows).
@@ -356,16 +369,17 @@ int fsie_moe_group(const int32_t* ids, int n_pairs, int experts, int tile_rows, 
                    int32_t* tiles, int max_tiles, hipStream_t stream);
 // One product per expert over its tiles: out[slot] = epilogue(A[row(slot)] . W[expert]^T), W [experts][N][K] in `dtype`.
 // gather_div > 0: row(slot) = order[slot] / gather_div (rows of A are tokens); 0: row(slot) = slot.
-// epilogue 0: exact GELU, out in `dtype`; 1: times slot_weight[order[slot]], out float32; 2 + a (a: FsieGateAct): the rows
-// of W[expert] are gate and up in turn (N even) and out [slots][N / 2] = act(gate) * up in `dtype`.  tile_rows: 16, 32, 64 or 128,
+// epilogue 0: exact GELU, out in `dtype`; 1: times slot_weight[order[slot]], out float32; 2 + a (a as for
+// fsie_gated_act, with limit and slope): the rows of W[expert] are gate and up in turn (N even) and out [slots][N / 2] = act(gate) * up in `dtype`.  tile_rows: 16, 32, 64 or 128,
 // the rows of a tile of `tiles`; fsie_moe_tile_rows names the one that suits a step of n_pairs pairs.
 int fsie_moe_tile_rows(int n_pairs, int experts);
 int fsie_moe_gemm(const void* a, const void* w, void* out, const int32_t* tiles, int max_tiles, const int32_t* order,
                   int gather_div, const float* pair_weight, int N, int K, int epilogue, int dtype, int tile_rows,
-                  hipStream_t stream);
-// y[t] = sum over the token's choices, in their order, of rows[slot_of[t * top + c]]; y float32 [n_tokens][hidden]
+                  float limit, float slope, hipStream_t stream);
+// y[t] = sum over the token's choices, in their order, of rows[slot_of[t * top + c]] (+ shared[t]); y float32
+// [n_tokens][hidden].  shared (or null): [n_tokens][hidden] of `dtype`, or shared_parts float32 arrays of that shape to add up.
 int fsie_moe_combine(const float* rows, const int32_t* slot_of, float* y, int n_tokens, int top, int hidden,
-                     hipStream_t stream);
+                     const void* shared, int shared_parts, int dtype, hipStream_t stream);
 
 #ifdef __cplusplus
 }

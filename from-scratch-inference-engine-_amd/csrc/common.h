@@ -64,6 +64,19 @@ __device__ __forceinline__ float gate_act(float g, int act) {
     return g / (1.0f + expf(-g));
 }
 
+// What a gated feed-forward multiplies: a FsieGateAct of the gate times the up value, or, 3: with the gate cut off above
+// at `limit` and the up value on both sides, g sigmoid(slope g) (u + 1).
+enum FsieGatePair { FSIE_PAIR_CLIPPED = 3 };
+#define FSIE_PAIR_KNOWN(act) (FSIE_ACT_KNOWN(act) || (act) == FSIE_PAIR_CLIPPED)
+__device__ __forceinline__ float gate_pair(float g, float u, int act, float limit, float slope) {
+    if (act == FSIE_PAIR_CLIPPED) {
+        g = fminf(g, limit);
+        u = fminf(fmaxf(u, -limit), limit);
+        return g / (1.0f + expf(-slope * g)) * (u + 1.0f);
+    }
+    return gate_act(g, act) * u;
+}
+
 // ---- activations of one value (a feed-forward without a gate) ------------------------------
 // 1: xIELU, z / 2 plus pos * z^2 above zero and neg * (exp(z) - 1 - z) below it.
 enum FsiePointAct { FSIE_POINT_NONE = 0, FSIE_POINT_XIELU = 1 };

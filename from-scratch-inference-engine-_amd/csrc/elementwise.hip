@@ -273,24 +273,36 @@ void launch_rmsnorm(const NormCall& c) {
     }
 }
 
-// out[t, j] = silu(x[t, 2j]) * x[t, 2j + 1]; x is [T, 2*inter] with gate and up interleaved.
+// out[t, j] = the product of the gate x[t, 2j] and the up value x[t, 2j + 1] (gate_pair); x is [T, 2*inter].
 template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ x, T* __restrict__ out, int64_t total, int inter, int act) {
+__global__ void swiglu_kernel(const T* __restrict__ x, T* __restrict__ out, int64_t total, int inter, int act, float limit,
+                              float slope) {
     const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (i >= total) return;
     const float g = to_float(x[2 * i]);
     const float u = to_float(x[2 * i + 1]);
-    out[i] = from_float<T>(gate_act(g, act) * u);
+    out[i] = from_float<T>(gate_pair(g, u, act, limit, slope));
 }
 
 // four outputs per thread: 8 inputs in 16 (bfloat16) or 32 (float32) bytes
 template <typename T>
-__global__ void swiglu_vec_kernel(const T* __restrict__ x, T* __restrict__ out, int64_t quads, int act) {
+__global__ void swiglu_vec_kernel(const T* __restrict__ x, T* __restrict__ out, int64_t quads, int act, float limit,
+                                  float slope) {
     const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (i >= quads) return;
     const float4 a = Pack4<T>::load(x + 8 * i), b = Pack4<T>::load(x + 8 * i + 4);
-    Pack4<T>::store(out + 4 * i, float4{gate_act(a.x, act) * a.y, gate_act(a.z, act) * a.w,
-                                        gate_act(b.x, act) * b.y, gate_act(b.z, act) * b.w});
+    Pack4<T>::store(out + 4 * i, float4{gate_pair(a.x, a.y, act, limit, slope), gate_pair(a.z, a.w, act, limit, slope),
+                                        gate_pair(b.x, b.y, act, limit, slope), gate_pair(b.z, b.w, act, limit, slope)});
+}
+
+// y[r][0 .. cols) = x[r][0 .. cols) rounded to T; rows of y are y_stride values apart.  grid = (rows, blocks of columns)
+template <typename T, bool VEC>
+__global__ void round_columns_kernel(const float* __restrict__ x, T* __restrict__ y, int64_t y_stride, int cols) {
+    const int64_t row = blockIdx.x;
+    const int j = (blockIdx.y * blockDim.x + threadIdx.x) * (VEC ? 4 : 1);
+    if (j >= cols) return;
+    if (VEC) Pack4<T>::store(y + row * y_stride + j, Pack4<float>::load(x + row * cols + j));
+    else y[row * y_stride + j] = from_float<T>(x[row * cols + j]);
 }
 
 template <typename T>
@@ -559,13 +571,13 @@ extern "C" int fsie_embedding(const void* table, int dtype, const int32_t* ids, 
     return 0;
 }
 
-// n_parts > 0: delta is n_parts float32 arrays [total_rows, hidden], one after the other, whose sum
+// n_parts > 0: delta is n_parts float32 arrays [total_rows, hidden] (one: an unrounded delta), one after the other, whose sum
 // (taken in order) is the delta; total_rows is the number of rows of the residual.
 extern "C" int fsie_rmsnorm(float* residual, const void* delta, const float* weight, void* out,
                             const int32_t* rows, int n_rows, int hidden, float eps, int dtype,
                             int write_back, int n_parts, int total_rows, hipStream_t stream) {
-    FSIE_REQUIRE(n_parts >= 0 && n_parts <= FSIE_GEMM_MAX_SPLITS && n_parts != 1,
-                 "rmsnorm: the delta comes whole or in 2..%d parts, not %d", FSIE_GEMM_MAX_SPLITS, n_parts);
+    FSIE_REQUIRE(n_parts >= 0 && n_parts <= FSIE_GEMM_MAX_SPLITS,
+                 "rmsnorm: the delta comes whole or in 1..%d float32 parts, not %d", FSIE_GEMM_MAX_SPLITS, n_parts);
     FSIE_REQUIRE(n_parts == 0 || (delta && total_rows > 0), "rmsnorm: parts without a delta or a row count");
     FSIE_REQUIRE(n_rows >= 0 && hidden > 0, "rmsnorm: bad sizes rows=%d H=%d", n_rows, hidden);
     FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "rmsnorm: unknown dtype %d", dtype);
@@ -583,9 +595,10 @@ extern "C" int fsie_rmsnorm(float* residual, const void* delta, const float* wei
     return 0;
 }
 
-extern "C" int fsie_gated_act(const void* x, void* out, int n_tokens, int inter, int dtype, int act, hipStream_t stream) {
+extern "C" int fsie_gated_act(const void* x, void* out, int n_tokens, int inter, int dtype, int act, float limit, float slope,
+                              hipStream_t stream) {
     FSIE_REQUIRE(n_tokens >= 0 && inter > 0, "swiglu: bad sizes T=%d I=%d", n_tokens, inter);
-    FSIE_REQUIRE(FSIE_ACT_KNOWN(act), "gated_act: unknown activation %d", act);
+    FSIE_REQUIRE(FSIE_PAIR_KNOWN(act), "gated_act: unknown activation %d", act);
     FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "swiglu: unknown dtype %d", dtype);
     const int64_t total = static_cast<int64_t>(n_tokens) * inter;
     if (total == 0) return 0;
@@ -593,18 +606,36 @@ extern "C" int fsie_gated_act(const void* x, void* out, int n_tokens, int inter,
     const int64_t work = vec ? total / 4 : total;
     const unsigned grid = static_cast<unsigned>(ceil_div64(work, kThreads));
     if (dtype == FSIE_F32) {
-        if (vec) swiglu_vec_kernel<float><<<grid, kThreads, 0, stream>>>(static_cast<const float*>(x), static_cast<float*>(out), work, act);
-        else swiglu_kernel<float><<<grid, kThreads, 0, stream>>>(static_cast<const float*>(x), static_cast<float*>(out), total, inter, act);
+        if (vec) swiglu_vec_kernel<float><<<grid, kThreads, 0, stream>>>(static_cast<const float*>(x), static_cast<float*>(out), work, act, limit, slope);
+        else swiglu_kernel<float><<<grid, kThreads, 0, stream>>>(static_cast<const float*>(x), static_cast<float*>(out), total, inter, act, limit, slope);
     } else {
-        if (vec) swiglu_vec_kernel<bf16_t><<<grid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<bf16_t*>(out), work, act);
-        else swiglu_kernel<bf16_t><<<grid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<bf16_t*>(out), total, inter, act);
+        if (vec) swiglu_vec_kernel<bf16_t><<<grid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<bf16_t*>(out), work, act, limit, slope);
+        else swiglu_kernel<bf16_t><<<grid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<bf16_t*>(out), total, inter, act, limit, slope);
     }
     FSIE_CHECK_LAUNCH("swiglu");
     return 0;
 }
 
 extern "C" int fsie_swiglu(const void* x, void* out, int n_tokens, int inter, int dtype, hipStream_t stream) {
-    return fsie_gated_act(x, out, n_tokens, inter, dtype, FSIE_ACT_SILU, stream);
+    return fsie_gated_act(x, out, n_tokens, inter, dtype, FSIE_ACT_SILU, 0.f, 0.f, stream);
+}
+
+extern "C" int fsie_round_columns(const float* x, void* y, int64_t y_stride, int rows, int cols, int dtype, hipStream_t stream) {
+    FSIE_REQUIRE(rows >= 0 && cols > 0 && y_stride >= cols && x && y, "round_columns: bad operands, %d x %d", rows, cols);
+    FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "round_columns: unknown dtype %d", dtype);
+    if (rows == 0) return 0;
+    const int64_t unit = 4 * (dtype == FSIE_F32 ? 4 : 2);
+    const bool vec = cols % 4 == 0 && y_stride % 4 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(y) % unit == 0;
+    const dim3 grid(static_cast<unsigned>(rows), static_cast<unsigned>(ceil_div64(vec ? cols / 4 : cols, kThreads)));
+#define FSIE_ROUND_COLUMNS(T, V) round_columns_kernel<T, V><<<grid, kThreads, 0, stream>>>(x, static_cast<T*>(y), y_stride, cols)
+    if (dtype == FSIE_F32) {
+        if (vec) FSIE_ROUND_COLUMNS(float, true); else FSIE_ROUND_COLUMNS(float, false);
+    } else {
+        if (vec) FSIE_ROUND_COLUMNS(bf16_t, true); else FSIE_ROUND_COLUMNS(bf16_t, false);
+    }
+#undef FSIE_ROUND_COLUMNS
+    FSIE_CHECK_LAUNCH("round_columns");
+    return 0;
 }
 
 extern "C" int fsie_round_to(const float* x, void* y, int64_t total, int dtype, hipStream_t stream) {

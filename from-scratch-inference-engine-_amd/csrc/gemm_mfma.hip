@@ -5,7 +5,7 @@
 // bfloat16 only.  M <= 64, K a multiple of 8, x and w 16-byte aligned.
 // waves (K split inside a workgroup) and blocks (16-row blocks of W per workgroup): 0 = choose.
 // epilogue: 0 = y = d (+ bias); 3 = the same as 1 with max(gate, 0) on the gate; 1 = SiLU*up over interleaved gate/up rows (N even, no bias, y is [M, N/2]);
-// 2 = the same with GELU (tanh form) for SiLU.
+// 2 = the same with GELU (tanh form) for SiLU; 4 = FSIE_PAIR_CLIPPED with act_pos, act_neg as limit and slope.
 // splits > 1: K is cut into that many slices, each summed by workgroups of its own; y is then
 // float32 [splits, M, N], partial sums without bias, which the consumer adds in the order of the slices
 // (fsie_rmsnorm takes them as its delta).  Every slice must hold at least 64 values of K.
@@ -20,7 +20,7 @@ static int gemm_mfma_skinny(const void* x, const void* w, const float* bias, voi
                  "gemm_mfma_skinny: partial sums are float32, without bias or epilogue");
     FSIE_REQUIRE(splits == 1 || ((K + splits - 1) / splits + 63) / 64 * 64 * (splits - 1) < K,
                  "gemm_mfma_skinny: K=%d is too short for %d slices", K, splits);
-    FSIE_REQUIRE(epilogue >= 0 && epilogue <= 3, "gemm_mfma_skinny: unknown epilogue %d", epilogue);
+    FSIE_REQUIRE(epilogue >= 0 && epilogue <= 4, "gemm_mfma_skinny: unknown epilogue %d", epilogue);
     FSIE_REQUIRE(epilogue == 0 || (N % 2 == 0 && !bias && !out_f32),
                  "gemm_mfma_skinny: the SiLU*up epilogue needs an even N, no bias and a bfloat16 result");
     FSIE_REQUIRE(M >= 0 && N > 0 && K > 0, "gemm_mfma_skinny: bad sizes M=%d N=%d K=%d", M, N, K);
@@ -63,7 +63,7 @@ static int gemm_mfma_skinny(const void* x, const void* w, const float* bias, voi
     if (mt * blocks > 4 && waves > 8) waves = 8;  // LDS of the reduction
     fsie_mm::Call call{x, w, bias, y, M, N, K, splits, stream, fsie_mm::RopeArgs{}};
     call.act_pos = act_pos, call.act_neg = act_neg;
-    call.act = epilogue == 0 ? point : epilogue == 3 ? FSIE_ACT_RELU : (epilogue == 2 ? FSIE_ACT_GELU_TANH : FSIE_ACT_SILU);
+    call.act = epilogue == 0 ? point : epilogue == 4 ? FSIE_PAIR_CLIPPED : epilogue == 3 ? FSIE_ACT_RELU : (epilogue == 2 ? FSIE_ACT_GELU_TANH : FSIE_ACT_SILU);
     if (epilogue != 0) return fsie_mm::launch_swiglu(blocks, waves, call);
     return out_f32 ? fsie_mm::launch_f32(mt, blocks, waves, call) : fsie_mm::launch_bf16(blocks, waves, call);
 }
@@ -71,6 +71,7 @@ static int gemm_mfma_skinny(const void* x, const void* w, const float* bias, voi
 extern "C" int fsie_gemm_mfma_skinny(const void* x, const void* w, const float* bias, void* y, int M, int N, int K,
                                      int out_f32, int waves, int blocks, int epilogue, int splits,
                                      hipStream_t stream) {
+    FSIE_REQUIRE(epilogue <= 3, "gemm_mfma_skinny: unknown epilogue %d", epilogue);
     return gemm_mfma_skinny(x, w, bias, y, M, N, K, out_f32, waves, blocks, epilogue, splits, FSIE_POINT_NONE, 0.f, 0.f, stream);
 }
 
@@ -78,6 +79,14 @@ extern "C" int fsie_gemm_mfma_skinny(const void* x, const void* w, const float* 
 extern "C" int fsie_gemm_mfma_skinny_act(const void* x, const void* w, const float* bias, void* y, int M, int N, int K,
                                          int waves, int blocks, int act, float act_pos, float act_neg, hipStream_t stream) {
     return gemm_mfma_skinny(x, w, bias, y, M, N, K, 0, waves, blocks, 0, 1, act, act_pos, act_neg, stream);
+}
+
+// y [M, N / 2] bfloat16 = the product of gate and up value (FsieGateAct or FsieGatePair) of w's rows in turn.
+extern "C" int fsie_gemm_mfma_skinny_gated(const void* x, const void* w, void* y, int M, int N, int K, int waves, int blocks,
+                                           int act, float limit, float slope, hipStream_t stream) {
+    FSIE_REQUIRE(FSIE_PAIR_KNOWN(act), "gemm_mfma_skinny_gated: unknown activation %d", act);
+    const int epilogue = act == FSIE_PAIR_CLIPPED ? 4 : act == FSIE_ACT_RELU ? 3 : act == FSIE_ACT_GELU_TANH ? 2 : 1;
+    return gemm_mfma_skinny(x, w, nullptr, y, M, N, K, 0, waves, blocks, epilogue, 1, FSIE_POINT_NONE, limit, slope, stream);
 }
 
 // The fused q/k/v projection of an attention layer with the position encoding in its epilogue:

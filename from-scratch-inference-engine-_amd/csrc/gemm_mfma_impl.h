@@ -58,7 +58,7 @@ __device__ __forceinline__ void rotation(double pos, double inv_freq, float* c, 
 // MT = tiles of 16 rows of X, NB = blocks of 16 rows of W per workgroup (they share the X
 // fragments), WAVES = waves of the workgroup, which split K.
 // EPI_SWIGLU: the rows of W are gate and up interleaved; the output has N/2 columns,
-// y[m, j] = silu(d[2j]) * d[2j + 1], computed in float32 from the accumulators.
+// y[m, j] = gate_pair(d[2j], d[2j + 1]), computed in float32 from the accumulators (act_pos, act_neg: its limit and slope).
 // EPI_ROPE: see RopeArgs.  The rows of W are taken in pairs (i, i + head_dim/2) of a head, numbered
 // through all heads; a workgroup owns `pairs_per_wg` consecutive pairs, eight to a block: tile rows
 // 0..7 are the first members, rows 8..15 the second, so that both members of a pair lie in one
@@ -282,7 +282,7 @@ __global__ __launch_bounds__(WAVES * FSIE_WAVE) void gemm_mfma_skinny_kernel(
                     const int nn = n0 + nb * 16 + kg * 4 + r;  // even: a gate row, nn + 1 its up row
                     if (nn + 1 < N) {
                         const float g = acc[nb][t][r], u = acc[nb][t][r + 1];
-                        y[static_cast<int64_t>(m) * (N / 2) + nn / 2] = from_float<OutT>(gate_act(g, act) * u);
+                        y[static_cast<int64_t>(m) * (N / 2) + nn / 2] = from_float<OutT>(gate_pair(g, u, act, act_pos, act_neg));
                     }
                 }
                 continue;
@@ -308,7 +308,7 @@ struct Call {
     int splits;  // slices of K, each a workgroup row of its own (partial sums out) when > 1
     hipStream_t stream;
     RopeArgs rope;
-    int act = 0;  // EPI_SWIGLU: the gate's activation (FsieGateAct); EPI_PLAIN with a bfloat16 result: FsiePointAct
+    int act = 0;  // EPI_SWIGLU: FsieGateAct or FsieGatePair; EPI_PLAIN with a bfloat16 result: FsiePointAct
     float act_pos = 0.f, act_neg = 0.f;  // its constants
 };
 

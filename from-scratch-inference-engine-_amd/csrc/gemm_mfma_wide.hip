@@ -67,7 +67,7 @@ struct PointEpilogue {
 // MT tiles of 16 rows of X; WAVES waves of NB blocks of 16 rows of W each per workgroup (a wave's
 // blocks share the B fragments it reads from LDS: with four tiles of X one block a wave would be
 // bound by those reads); STEPS 32-wide MFMA steps per stage (KS = 32 * STEPS values of K).
-// GATED: the rows of W are gate and up interleaved and y is bfloat16 [M, N / 2], silu(gate) * up
+// GATED: the rows of W are gate and up interleaved and y is bfloat16 [M, N / 2], gate_pair (point.pos, point.neg: its constants)
 // from the accumulators (a lane holds rows 4 kg .. 4 kg + 3 of a block: two pairs); one slice only.
 template <int MT, int WAVES, int STEPS, int NB, int RESULT, bool FRAGS>
 __global__ __launch_bounds__(WAVES * 64) void gemm_mfma_wide_kernel(const bf16_t* __restrict__ x,
@@ -203,7 +203,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_mfma_wide_kernel(const bf16_t
                 if (m >= M || nn >= N) continue;      // N is a multiple of 4 here (checked by the host)
                 const float g0 = acc[nb][t][0], u0 = acc[nb][t][1], g1 = acc[nb][t][2], u1 = acc[nb][t][3];
                 out[(static_cast<int64_t>(m) * (N / 2) + nn / 2) / 2] =
-                    pack2_bf16(gate_act(g0, act) * u0, gate_act(g1, act) * u1);
+                    pack2_bf16(gate_pair(g0, u0, act, point.pos, point.neg), gate_pair(g1, u1, act, point.pos, point.neg));
             }
         return;
     }
@@ -475,10 +475,11 @@ extern "C" int fsie_gemm_mfma_wide(const void* x, const void* w, float* y, int M
 
 // The same product with the rows of w as gate and up in turn: y is bfloat16 [M, N / 2], silu(gate) * up.
 // N a multiple of 4; one slice of K.
-// act: the gate's activation (FsieGateAct: 0 SiLU, 1 GELU in its tanh form).
+// act: FsieGateAct or FsieGatePair with its limit and slope.
 extern "C" int fsie_gemm_mfma_wide_gated(const void* x, const void* w, void* y, int M, int N, int K, int waves,
-                                         int blocks, int frags, int act, hipStream_t stream) {
-    FSIE_REQUIRE(FSIE_ACT_KNOWN(act), "gemm_mfma_wide_gated: unknown activation %d", act);
+                                         int blocks, int frags, int act, float limit, float slope,
+                                         hipStream_t stream) {
+    FSIE_REQUIRE(FSIE_PAIR_KNOWN(act), "gemm_mfma_wide_gated: unknown activation %d", act);
     FSIE_REQUIRE(M >= 0 && N > 0 && K > 0, "gemm_mfma_wide_swiglu: bad sizes M=%d N=%d K=%d", M, N, K);
     FSIE_REQUIRE(M <= (frags ? FSIE_GEMM_MFMA_WIDE_MAX_M : FSIE_GEMM_MFMA_SKINNY_MAX_M),
                  "gemm_mfma_wide_swiglu: at most %d rows (%d on a fragment-ordered weight), got %d",
@@ -498,8 +499,10 @@ extern "C" int fsie_gemm_mfma_wide_gated(const void* x, const void* w, void* y, 
     const bf16_t* xp = static_cast<const bf16_t*>(x);
     const bf16_t* wq = static_cast<const bf16_t*>(w);
     float* yp = static_cast<float*>(y);
-    if (frags) return launch_shape_of<GATED, true>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, act, PointEpilogue{}, stream);
-    return launch_shape_of<GATED, false>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, act, PointEpilogue{}, stream);
+    PointEpilogue pair;
+    pair.pos = limit, pair.neg = slope;
+    if (frags) return launch_shape_of<GATED, true>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, act, pair, stream);
+    return launch_shape_of<GATED, false>(mt, waves, blocks, xp, wq, yp, M, N, K, 1, k_slice, act, pair, stream);
 }
 
 // y = act(x . w^T + bias) in bfloat16 [M, N], act a FsiePointAct: one slice of K, N a multiple of 4.
@@ -538,7 +541,7 @@ extern "C" int fsie_gemm_mfma_wide_act_takes(int M, int N, int K) {
 
 extern "C" int fsie_gemm_mfma_wide_swiglu(const void* x, const void* w, void* y, int M, int N, int K, int waves,
                                           int blocks, int frags, hipStream_t stream) {
-    return fsie_gemm_mfma_wide_gated(x, w, y, M, N, K, waves, blocks, frags, FSIE_ACT_SILU, stream);
+    return fsie_gemm_mfma_wide_gated(x, w, y, M, N, K, waves, blocks, frags, FSIE_ACT_SILU, 0.f, 0.f, stream);
 }
 
 // The copy of a bfloat16 matrix w [N, K] in the order of the matrix instruction's A fragments, for

@@ -9,7 +9,8 @@
 // themselves, every head reading the same keys, with queries [q~_h | rotated q part] of `width` values,
 // and W_uv,h is applied to its result.  The kernels here: what is written into the cache
 // (fsie_latent_prep), the rotation of pairs of neighbours (fsie_rope_pairs), and the product with a
-// matrix of its own for every head (fsie_head_gemm).
+// matrix of its own for every head (fsie_head_gemm), which also turns the heads' rotated parts beside it and
+// multiplies its results by gates.
 #include "common.h"
 #include "api.h"
 
@@ -39,7 +40,7 @@ __device__ __forceinline__ float rotated_neighbour(const T* __restrict__ run, in
 // One workgroup a token.  proj [tokens][stride] holds, of every token: the query latent (q_rank values
 // from dq_off), the key/value latent and the shared key part (kv_rank + rot_dim values from dkv_off), and
 // one gate a head (from g_off).
-//   cq[t]   = RMS norm of the query latent, weight q_weight                       (type T)
+//   cq[t]   = RMS norm of the query latent, weight q_weight                       (type T; q_rank 0: there is none)
 //   gate[t] = sigmoid of the gates                                                 (float32)
 //   cache row of the token (if the layer keeps a cache): [RMS norm of the latent, weight kv_weight |
 //             shared key part, its first 2 * pairs values rotated | zeros up to width]
@@ -52,7 +53,7 @@ __global__ __launch_bounds__(kThreads) void latent_prep_kernel(
     __shared__ float scratch[16];
     const int t = blockIdx.x;
     const T* row = proj + static_cast<int64_t>(t) * stride;
-    {
+    if (q_rank > 0) {
         const T* x = row + dq_off;
         float sum = 0.f;
         for (int j = threadIdx.x; j < q_rank; j += kThreads) sum += to_float(x[j]) * to_float(x[j]);
@@ -98,17 +99,56 @@ __global__ __launch_bounds__(kThreads) void rope_pairs_kernel(const T* __restric
     }
 }
 
-// y[t][h][n] = (sum over k of x[t][h][k] * w[h][n][k]) * (gate ? gate[t][h] : 1): a tile of 32 tokens by 64
+// What a product per head does beside its sums.  gate: float32 [tokens][heads], a factor a head.  gate_rows: logits of
+// the activations' type, gate_stride values a token, one for every output (head h's from h * N): their sigmoids are
+// factors.  rot_out_width > 0: the last block of the grid's first dimension turns the run of rot_width values at
+// x[t][h][rot_in ..] (|rot_pairs| pairs, see rotated_neighbour) into y[t][h][rot_out .. rot_out + rot_out_width), zeros at
+// its end.
+template <typename T>
+struct HeadExtras {
+    const float* gate;
+    const T* gate_rows;
+    int64_t gate_stride;
+    const float2* cos_sin;
+    int rot_in, rot_out, rot_width, rot_pairs, rot_out_width;
+};
+
+template <typename T>
+__device__ __forceinline__ void turn_heads(const HeadExtras<T>& ex, const T* __restrict__ x, int64_t x_stride, int x_first,
+                                           T* __restrict__ y, int64_t y_stride, int y_first, int t0, int tokens) {
+    const int n = ex.rot_pairs < 0 ? -ex.rot_pairs : ex.rot_pairs;
+    for (int e = threadIdx.x; e < tokens * ex.rot_out_width; e += kThreads) {
+        const int i = e / ex.rot_out_width, j = e - i * ex.rot_out_width;
+        const int64_t t = t0 + i;
+        const float v = j < ex.rot_width
+                            ? rotated_neighbour(x + t * x_stride + x_first + ex.rot_in, j, ex.rot_pairs, ex.cos_sin + t * n)
+                            : 0.f;
+        y[t * y_stride + y_first + ex.rot_out + j] = from_float<T>(v);
+    }
+}
+
+template <typename T>
+__device__ __forceinline__ float head_factor(const HeadExtras<T>& ex, int64_t t, int h, int heads, int64_t column) {
+    float g = ex.gate ? ex.gate[t * heads + h] : 1.0f;
+    if (ex.gate_rows) g *= 1.0f / (1.0f + expf(-to_float(ex.gate_rows[t * ex.gate_stride + column])));
+    return g;
+}
+
+// y[t][h][n] = (sum over k of x[t][h][k] * w[h][n][k]) * factor (HeadExtras): a tile of 32 tokens by 64
 // outputs of one head a workgroup, 32 values of k a pass through LDS, float32 sums.
 constexpr int kTileM = 32, kTileN = 64, kTileK = 32;
 template <typename T>
 __global__ __launch_bounds__(kThreads) void head_gemm_kernel(const T* __restrict__ x, int64_t x_stride, int x_off, int x_hs,
                                                              const T* __restrict__ w, T* __restrict__ y, int64_t y_stride,
-                                                             int y_off, int y_hs, const float* __restrict__ gate,
+                                                             int y_off, int y_hs, HeadExtras<T> ex,
                                                              int n_tokens, int heads, int N, int K) {
     __shared__ float xs[kTileM][kTileK + 1];
     __shared__ float ws[kTileN][kTileK + 1];
     const int h = blockIdx.z, n0 = blockIdx.x * kTileN, t0 = blockIdx.y * kTileM;
+    if (ex.rot_out_width && blockIdx.x == gridDim.x - 1) {
+        turn_heads(ex, x, x_stride, x_off + h * x_hs, y, y_stride, y_off + h * y_hs, t0, min(kTileM, n_tokens - t0));
+        return;
+    }
     const int tid = threadIdx.x, ty = tid >> 4, tx = tid & 15;
     const T* wh = w + static_cast<int64_t>(h) * N * K;
     float acc[2][4] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
@@ -140,11 +180,12 @@ __global__ __launch_bounds__(kThreads) void head_gemm_kernel(const T* __restrict
     for (int a = 0; a < 2; ++a) {
         const int t = t0 + 2 * ty + a;
         if (t >= n_tokens) continue;
-        const float g = gate ? gate[static_cast<int64_t>(t) * heads + h] : 1.0f;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx + 16 * j;
-            if (n < N) y[static_cast<int64_t>(t) * y_stride + y_off + h * y_hs + n] = from_float<T>(acc[a][j] * g);
+            if (n < N)
+                y[static_cast<int64_t>(t) * y_stride + y_off + h * y_hs + n] =
+                    from_float<T>(acc[a][j] * head_factor(ex, t, h, heads, static_cast<int64_t>(h) * N + n));
         }
     }
 }
@@ -167,10 +208,14 @@ template <int MT>
 __global__ __launch_bounds__(kThreads) void head_gemm_mfma_kernel(const bf16_t* __restrict__ x, int64_t x_stride, int x_off,
                                                                   int x_hs, const bf16_t* __restrict__ w,
                                                                   bf16_t* __restrict__ y, int64_t y_stride, int y_off,
-                                                                  int y_hs, const float* __restrict__ gate, int n_tokens,
+                                                                  int y_hs, HeadExtras<bf16_t> ex, int n_tokens,
                                                                   int heads, int N, int K) {
     const int h = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n0 = (blockIdx.x * 4 + wave) * 64, t0 = blockIdx.y * (16 * MT);
+    if (ex.rot_out_width && blockIdx.x == gridDim.x - 1) {
+        turn_heads(ex, x, x_stride, x_off + h * x_hs, y, y_stride, y_off + h * y_hs, t0, min(16 * MT, n_tokens - t0));
+        return;
+    }
     if (n0 >= N) return;
     const int r = lane & 15, kq = (lane >> 4) * 8;
     const bf16_t* wh = w + static_cast<int64_t>(h) * N * K;
@@ -216,14 +261,14 @@ __global__ __launch_bounds__(kThreads) void head_gemm_mfma_kernel(const bf16_t* 
     for (int b = 0; b < MT; ++b) {
         const int t = t0 + 16 * b + r;
         if (t >= n_tokens) continue;
-        const float g = gate ? gate[static_cast<int64_t>(t) * heads + h] : 1.0f;
         bf16_t* dst = y + static_cast<int64_t>(t) * y_stride + y_off + h * y_hs;
 #pragma unroll
         for (int a = 0; a < 4; ++a) {
             const int n = n0 + 16 * a + nq;
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                if (n + i < N) dst[n + i] = from_float<bf16_t>(acc[a][b][i] * g);
+                if (n + i < N)
+                    dst[n + i] = from_float<bf16_t>(acc[a][b][i] * head_factor(ex, t, h, heads, static_cast<int64_t>(h) * N + n + i));
             }
         }
     }
@@ -236,10 +281,10 @@ extern "C" int fsie_latent_prep(const void* proj, int64_t stride, int dq_off, in
                                 const float* kv_weight, float eps, const float* cos_sin, void* cq, float* gate,
                                 const int32_t* slots, void* k_pool, void* v_pool, int width, int page_size,
                                 int64_t pool_slots, int n_tokens, int dtype, hipStream_t stream) {
-    FSIE_REQUIRE(n_tokens >= 0 && q_rank > 0 && kv_rank > 0 && rot_dim >= 0 && heads >= 0, "latent_prep: bad sizes");
+    FSIE_REQUIRE(n_tokens >= 0 && q_rank >= 0 && kv_rank > 0 && rot_dim >= 0 && heads >= 0, "latent_prep: bad sizes");
     FSIE_REQUIRE(2 * abs(rot_pairs) <= rot_dim, "latent_prep: %d rotated pairs do not fit %d values", rot_pairs, rot_dim);
     FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "latent_prep: unknown dtype %d", dtype);
-    FSIE_REQUIRE(proj && q_weight && cq && (gate || heads == 0), "latent_prep: missing operand");
+    FSIE_REQUIRE(proj && (q_rank == 0 || (q_weight && cq)) && (gate || heads == 0), "latent_prep: missing operand");
     FSIE_REQUIRE(dq_off >= 0 && dq_off + q_rank <= stride && g_off >= 0 && g_off + heads <= stride,
                  "latent_prep: the columns do not fit a row of %lld", static_cast<long long>(stride));
     const bool writes = k_pool != nullptr;
@@ -287,44 +332,60 @@ extern "C" int fsie_rope_pairs(const void* in, int64_t in_stride, int in_off, in
 }
 
 // x [n_tokens][x_stride]: head h's K values start at column x_off + h * x_hs; w [heads][N][K]; y likewise
-// with N values a head from y_off + h * y_hs; gate (or null) float32 [n_tokens][heads].
+// with N values a head from y_off + h * y_hs; gate (or null) float32 [n_tokens][heads]; gate_rows and the rotated runs:
+// see HeadExtras (columns rot_in and rot_out count from the head's first in x and in y).
 extern "C" int fsie_head_gemm(const void* x, int64_t x_stride, int x_off, int x_hs, const void* w, void* y, int64_t y_stride,
-                              int y_off, int y_hs, const float* gate, int n_tokens, int heads, int N, int K, int dtype,
-                              hipStream_t stream) {
+                              int y_off, int y_hs, const float* gate, const void* gate_rows, int64_t gate_stride, int rot_in,
+                              int rot_out, int rot_width, int rot_pairs, int rot_out_width, const float* cos_sin, int n_tokens,
+                              int heads, int N, int K, int dtype, hipStream_t stream) {
     FSIE_REQUIRE(n_tokens >= 0 && heads > 0 && heads <= 65535 && N > 0 && K > 0, "head_gemm: bad sizes T=%d heads=%d N=%d K=%d",
                  n_tokens, heads, N, K);
     FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "head_gemm: unknown dtype %d", dtype);
     FSIE_REQUIRE(x && w && y, "head_gemm: missing operand");
     FSIE_REQUIRE(x_off >= 0 && y_off >= 0 && x_off + (heads - 1) * x_hs + K <= x_stride && y_off + (heads - 1) * y_hs + N <= y_stride,
                  "head_gemm: the heads do not fit the rows");
+    FSIE_REQUIRE(!gate_rows || gate_stride >= static_cast<int64_t>(heads) * N, "head_gemm: a gate row is shorter than the heads");
+    FSIE_REQUIRE(rot_out_width >= 0 && rot_width >= 0 && rot_width <= rot_out_width && 2 * abs(rot_pairs) <= rot_width,
+                 "head_gemm: bad rotated run of %d values, %d pairs, %d places", rot_width, rot_pairs, rot_out_width);
+    if (rot_out_width) {
+        FSIE_REQUIRE((rot_pairs == 0 || cos_sin) && reinterpret_cast<uintptr_t>(cos_sin) % 8 == 0, "head_gemm: no cosines and sines");
+        FSIE_REQUIRE(rot_in >= 0 && x_off + (heads - 1) * x_hs + rot_in + rot_width <= x_stride && rot_out >= N &&
+                         y_off + (heads - 1) * y_hs + rot_out + rot_out_width <= y_stride,
+                     "head_gemm: the rotated runs do not fit the rows (or lie over the products)");
+    }
     if (n_tokens == 0) return 0;
+    const float2* cs = reinterpret_cast<const float2*>(cos_sin);
+    const unsigned turned = rot_out_width ? 1 : 0;  // one more block of the first dimension
     const int row_tiles = (n_tokens + kTileM - 1) / kTileM;
     FSIE_REQUIRE(row_tiles <= 65535, "head_gemm: %d tokens are more than one launch takes", n_tokens);
-    const dim3 grid((N + kTileN - 1) / kTileN, row_tiles, heads);
+    const dim3 grid((N + kTileN - 1) / kTileN + turned, row_tiles, heads);
     const bool aligned = K % 8 == 0 && x_stride % 8 == 0 && x_off % 8 == 0 && x_hs % 8 == 0 &&
                          reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0;
     if (dtype == FSIE_BF16 && aligned) {
         const bool two = n_tokens > 16;
         const int token_tiles = (n_tokens + (two ? 32 : 16) - 1) / (two ? 32 : 16);
         FSIE_REQUIRE(token_tiles <= 65535, "head_gemm: %d tokens are more than one launch takes", n_tokens);
-        const dim3 mgrid((N + 255) / 256, token_tiles, heads);
+        const dim3 mgrid((N + 255) / 256 + turned, token_tiles, heads);
+        const HeadExtras<bf16_t> ex{gate, static_cast<const bf16_t*>(gate_rows), gate_stride, cs, rot_in, rot_out, rot_width, rot_pairs, rot_out_width};
         if (two) {
             head_gemm_mfma_kernel<2><<<mgrid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), x_stride, x_off, x_hs,
                                                                     static_cast<const bf16_t*>(w), static_cast<bf16_t*>(y),
-                                                                    y_stride, y_off, y_hs, gate, n_tokens, heads, N, K);
+                                                                    y_stride, y_off, y_hs, ex, n_tokens, heads, N, K);
         } else {
             head_gemm_mfma_kernel<1><<<mgrid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), x_stride, x_off, x_hs,
                                                                     static_cast<const bf16_t*>(w), static_cast<bf16_t*>(y),
-                                                                    y_stride, y_off, y_hs, gate, n_tokens, heads, N, K);
+                                                                    y_stride, y_off, y_hs, ex, n_tokens, heads, N, K);
         }
     } else if (dtype == FSIE_F32) {
+        const HeadExtras<float> ex{gate, static_cast<const float*>(gate_rows), gate_stride, cs, rot_in, rot_out, rot_width, rot_pairs, rot_out_width};
         head_gemm_kernel<float><<<grid, kThreads, 0, stream>>>(static_cast<const float*>(x), x_stride, x_off, x_hs,
                                                              static_cast<const float*>(w), static_cast<float*>(y), y_stride,
-                                                             y_off, y_hs, gate, n_tokens, heads, N, K);
+                                                             y_off, y_hs, ex, n_tokens, heads, N, K);
     } else {
+        const HeadExtras<bf16_t> ex{gate, static_cast<const bf16_t*>(gate_rows), gate_stride, cs, rot_in, rot_out, rot_width, rot_pairs, rot_out_width};
         head_gemm_kernel<bf16_t><<<grid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), x_stride, x_off, x_hs,
                                                               static_cast<const bf16_t*>(w), static_cast<bf16_t*>(y), y_stride,
-                                                              y_off, y_hs, gate, n_tokens, heads, N, K);
+                                                              y_off, y_hs, ex, n_tokens, heads, N, K);
     }
     FSIE_CHECK_LAUNCH("head_gemm");
     return 0;

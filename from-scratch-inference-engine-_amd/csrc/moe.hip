@@ -246,7 +246,7 @@ template <typename T, int MT, int NB, bool KSPLIT>
 __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ a, const T* __restrict__ w, void* __restrict__ out,
                                                        const int32_t* __restrict__ tiles, const int32_t* __restrict__ order,
                                                        int gather_div, const float* __restrict__ pair_weight, int N, int K,
-                                                       int epilogue, int max_tiles) {
+                                                       int epilogue, int max_tiles, float limit, float slope) {
     __shared__ float red[KSPLIT ? 3 * MT * NB * 4 * 64 : 1];
     int tile, n_block;
     constexpr int kOutputs = KSPLIT ? 16 * NB : 64 * NB;  // outputs a workgroup
@@ -393,7 +393,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ a, 
                 } else if (epilogue >= 2) {
                     // gate and up rows in turn: the even output's neighbour lane holds its up value
                     const float up = __shfl_xor(v, 1, FSIE_WAVE);
-                    if (!(n & 1)) static_cast<T*>(out)[slot * (N / 2) + n / 2] = from_float<T>(gate_act(v, epilogue - 2) * up);
+                    if (!(n & 1)) static_cast<T*>(out)[slot * (N / 2) + n / 2] = from_float<T>(gate_pair(v, up, epilogue - 2, limit, slope));
                 } else {
                     static_cast<T*>(out)[slot * N + n] = from_float<T>(gelu_erf(v));
                 }
@@ -402,10 +402,22 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ a, 
     }
 }
 
-// grid = (tokens, blocks of 1024 values); VEC: four values a thread
-template <bool VEC>
+// grid = (tokens, blocks of 1024 values); VEC: four values a thread.  shared (or null): rows of an expert that every token
+// takes, added last: SharedT values [tokens][hidden], or with shared_parts > 0 that many float32 arrays of them, one
+// after the other, added up first.
+template <typename SharedT>
+__device__ __forceinline__ float shared_value(const void* shared, int shared_parts, int64_t plane, int64_t at) {
+    if (shared_parts == 0) return to_float(static_cast<const SharedT*>(shared)[at]);
+    const float* p = static_cast<const float*>(shared) + at;
+    float v = p[0];
+    for (int s = 1; s < shared_parts; ++s) v += p[s * plane];
+    return v;
+}
+
+template <typename SharedT, bool VEC>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ rows, const int32_t* __restrict__ slot_of,
-                                                          float* __restrict__ y, int top, int hidden) {
+                                                          float* __restrict__ y, int top, int hidden,
+                                                          const void* __restrict__ shared, int shared_parts, int64_t plane) {
     const int t = blockIdx.x;
     int slots[kMaxTop];
 #pragma unroll
@@ -429,6 +441,11 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
         }
     }
     float* dst = y + static_cast<int64_t>(t) * hidden + j;
+    if (shared) {
+#pragma unroll
+        for (int u = 0; u < V; ++u)
+            sum[u] += shared_value<SharedT>(shared, shared_parts, plane, static_cast<int64_t>(t) * hidden + j + u);
+    }
     if constexpr (VEC) *reinterpret_cast<float4*>(dst) = float4{sum[0], sum[1], sum[2], sum[3]};
     else dst[0] = sum[0];
 }
@@ -484,12 +501,12 @@ extern "C" int fsie_moe_tile_rows(int n_pairs, int experts) {
 
 extern "C" int fsie_moe_gemm(const void* a, const void* w, void* out, const int32_t* tiles, int max_tiles,
                              const int32_t* order, int gather_div, const float* pair_weight, int N, int K, int epilogue,
-                             int dtype, int tile_rows, hipStream_t stream) {
+                             int dtype, int tile_rows, float limit, float slope, hipStream_t stream) {
     FSIE_REQUIRE(max_tiles >= 0 && N > 0 && K > 0 && gather_div >= 0, "moe_gemm: bad sizes tiles=%d N=%d K=%d", max_tiles, N, K);
     FSIE_REQUIRE(tile_rows == 16 || tile_rows == 32 || tile_rows == 64 || tile_rows == 128,
                  "moe_gemm: tiles of %d rows (the kernels take 16, 32, 64, 128)", tile_rows);
     FSIE_REQUIRE(a && w && out && tiles && order, "moe_gemm: missing operand");
-    FSIE_REQUIRE(epilogue == 0 || (epilogue == 1 && pair_weight) || (epilogue >= 2 && FSIE_ACT_KNOWN(epilogue - 2) && N % 2 == 0),
+    FSIE_REQUIRE(epilogue == 0 || (epilogue == 1 && pair_weight) || (epilogue >= 2 && FSIE_PAIR_KNOWN(epilogue - 2) && N % 2 == 0),
                  "moe_gemm: unknown epilogue %d", epilogue);
     FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "moe_gemm: unknown dtype %d", dtype);
     if (max_tiles == 0) return 0;
@@ -499,7 +516,7 @@ extern "C" int fsie_moe_gemm(const void* a, const void* w, void* out, const int3
     moe_gemm_kernel<T, MT, NB, KSPLIT><<<static_cast<unsigned>((KSPLIT ? max_tiles : per_die * 8) *                        \
                                                                ceil_div64(N, KSPLIT ? 16 * NB : 64 * NB)),                  \
                                          256, 0, stream>>>(static_cast<const T*>(a), static_cast<const T*>(w), out, tiles, order, \
-                                                           gather_div, pair_weight, N, K, epilogue, max_tiles)
+                                                           gather_div, pair_weight, N, K, epilogue, max_tiles, limit, slope)
 #define FSIE_MOE_GEMM_T(T)                                      \
     if (tile_rows == 16) FSIE_MOE_GEMM(T, 1, 2, true);          \
     else if (tile_rows == 32) FSIE_MOE_GEMM(T, 2, 2, true);     \
@@ -513,15 +530,23 @@ extern "C" int fsie_moe_gemm(const void* a, const void* w, void* out, const int3
 }
 
 extern "C" int fsie_moe_combine(const float* rows, const int32_t* slot_of, float* y, int n_tokens, int top, int hidden,
-                                hipStream_t stream) {
+                                const void* shared, int shared_parts, int dtype, hipStream_t stream) {
     FSIE_REQUIRE(n_tokens >= 0 && top > 0 && hidden > 0, "moe_combine: bad sizes");
+    FSIE_REQUIRE(shared_parts >= 0 && shared_parts <= FSIE_GEMM_MAX_SPLITS, "moe_combine: %d partial sums", shared_parts);
+    FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "moe_combine: unknown dtype %d", dtype);
     FSIE_REQUIRE(rows && slot_of && y, "moe_combine: missing operand");
     if (n_tokens == 0) return 0;
     FSIE_REQUIRE(top <= kMaxTop, "moe_combine: top %d (at most %d)", top, kMaxTop);
     const bool vec = hidden % 4 == 0 && (reinterpret_cast<uintptr_t>(rows) & 15) == 0 && (reinterpret_cast<uintptr_t>(y) & 15) == 0;
     const dim3 grid(n_tokens, static_cast<unsigned>(ceil_div64(hidden, vec ? 1024 : 256)));
-    if (vec) moe_combine_kernel<true><<<grid, 256, 0, stream>>>(rows, slot_of, y, top, hidden);
-    else moe_combine_kernel<false><<<grid, 256, 0, stream>>>(rows, slot_of, y, top, hidden);
+    const int64_t plane = static_cast<int64_t>(n_tokens) * hidden;
+#define FSIE_COMBINE(T, V) moe_combine_kernel<T, V><<<grid, 256, 0, stream>>>(rows, slot_of, y, top, hidden, shared, shared_parts, plane)
+    if (dtype == FSIE_F32) {
+        if (vec) FSIE_COMBINE(float, true); else FSIE_COMBINE(float, false);
+    } else {
+        if (vec) FSIE_COMBINE(bf16_t, true); else FSIE_COMBINE(bf16_t, false);
+    }
+#undef FSIE_COMBINE
     FSIE_CHECK_LAUNCH("moe_combine");
     return 0;
 }

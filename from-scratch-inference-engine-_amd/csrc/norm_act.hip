@@ -139,6 +139,42 @@ __global__ __launch_bounds__(THREADS) void sandwich_norm_vec_kernel(
     }
 }
 
+// One workgroup a row.  v = residual[row] + what is pending: nothing (delta null), y itself (post_weight null) or the RMS
+// norm of y, with y = delta[row] (one array of T, or the sum in order of n_parts float32 arrays).
+//   out[row][0 .. hidden) = v rounded to T (rows out_stride values apart);  residual[row] = restart[0 .. hidden)
+// The stream goes out and starts again from `restart`: what comes next is a delta on that.
+template <typename T>
+__global__ __launch_bounds__(kThreads) void stream_out_kernel(float* __restrict__ residual, const T* __restrict__ delta,
+                                                              const float* __restrict__ post_weight, float post_eps,
+                                                              T* __restrict__ out, int64_t out_stride,
+                                                              const float* __restrict__ restart, int hidden, int n_parts,
+                                                              int64_t part_stride) {
+    extern __shared__ float row_buf[];
+    __shared__ float scratch[16];
+    const int64_t row = blockIdx.x;
+    float* res = residual + row * hidden;
+    const float* parts = n_parts ? reinterpret_cast<const float*>(delta) + row * hidden : nullptr;
+    T* dst = out + row * out_stride;
+    float post_scale = 1.f;
+    if (delta) {
+        float sum_sq = 0.f;
+        for (int j = threadIdx.x; j < hidden; j += kThreads) {  // (a thread reads back only what it wrote itself)
+            float y = parts ? parts[j] : to_float(delta[row * hidden + j]);
+#pragma unroll 4
+            for (int s = 1; s < n_parts; ++s) y += parts[s * part_stride + j];
+            row_buf[j] = y;
+            sum_sq += y * y;
+        }
+        if (post_weight) post_scale = 1.0f / sqrtf(block_sum(sum_sq, scratch) / static_cast<float>(hidden) + post_eps);
+    }
+    for (int j = threadIdx.x; j < hidden; j += kThreads) {
+        float v = res[j];
+        if (delta) v += post_weight ? (row_buf[j] * post_scale) * post_weight[j] : row_buf[j];
+        dst[j] = from_float<T>(v);
+        res[j] = restart[j];
+    }
+}
+
 // One wave per (token, head): o [tokens][heads * width] float32 is normalised over the `width` values of
 // the head (plain weight [width], shared by the heads) and multiplied by act(gate) of the same place;
 // gate [tokens][gate_stride] of T (the columns of the head start at h * width).
@@ -236,6 +272,27 @@ extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const floa
                                                                       hidden, write_back, n_parts, part_stride);
     }
     FSIE_CHECK_LAUNCH("sandwich_norm");
+    return 0;
+}
+
+extern "C" int fsie_stream_out(float* residual, const void* delta, const float* post_weight, float post_eps, void* out,
+                               int64_t out_stride, const float* restart, int n_rows, int hidden, int dtype, int n_parts,
+                               hipStream_t stream) {
+    FSIE_REQUIRE(n_rows >= 0 && hidden > 0 && hidden <= 16384, "stream_out: bad sizes rows=%d hidden=%d (at most 16384)", n_rows, hidden);
+    FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "stream_out: unknown dtype %d", dtype);
+    FSIE_REQUIRE(residual && out && restart && out_stride >= hidden, "stream_out: missing operand");
+    FSIE_REQUIRE(n_parts >= 0 && n_parts <= FSIE_GEMM_MAX_SPLITS && (delta || (!n_parts && !post_weight)),
+                 "stream_out: %d partial sums, or a norm or sums of nothing", n_parts);
+    if (n_rows == 0) return 0;
+    const size_t lds = delta ? sizeof(float) * hidden : 0;
+    const int64_t part_stride = static_cast<int64_t>(n_rows) * hidden;
+    if (dtype == FSIE_F32)
+        stream_out_kernel<float><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const float*>(delta), post_weight, post_eps,
+                                                                    static_cast<float*>(out), out_stride, restart, hidden, n_parts, part_stride);
+    else
+        stream_out_kernel<bf16_t><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const bf16_t*>(delta), post_weight, post_eps,
+                                                                     static_cast<bf16_t*>(out), out_stride, restart, hidden, n_parts, part_stride);
+    FSIE_CHECK_LAUNCH("stream_out");
     return 0;
 }
 

@@ -75,6 +75,7 @@ class Model:
         self.dtype = resolve_dtype(dtype)
         self.device = torch.device(device)
         self.weight_bytes = 0
+        self.entrances = spec.entrances()
         # caches: one per call of the schedule that keeps one
         self.call_cache: List[int] = []
         needs: Dict[object, object] = {}
@@ -224,7 +225,11 @@ class Model:
         storage.clear_fresh(ctx)   # and the pages taken from the pools for this step hold nothing of their last owner
         kept = storage.view(EMBEDDING_CACHE, ctx, writes=True) if EMBEDDING_CACHE in self.cached_calls else None
         hidden = HiddenState(spec.embedding.embed(ctx, kept))
+        for entrance in self.entrances:
+            entrance.begin(hidden, ctx)
         for i, call in enumerate(spec.schedule):
+            if call.entrance is not None:
+                call.entrance.forward(hidden, ctx, call.entrance_number)
             cid = self.call_cache[i]
             cache = self._cache_view(storage, cid, ctx, call.cache_of is None) if cid in self.cached_calls else None
             own = block_state_cache(i)

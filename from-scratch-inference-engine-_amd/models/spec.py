@@ -5,7 +5,7 @@ from __future__ import annotations
 from dataclasses import dataclass, field
 from typing import Dict, List, Optional, Sequence
 
-from ..parts.base import Block, Norm, Part
+from ..parts.base import Block, Entrance, Norm, Part
 from ..parts.embedding import LMHead, TokenEmbedding
 from ..weights.loader import ParamBinding, TensorSpec
 
@@ -17,10 +17,13 @@ class LayerCall:
     ``layer`` indexes ``ModelSpec.layers`` (the same layer may be named by several calls: its
     weights are then shared, each call has a cache of its own).  ``cache_of`` = index of an
     *earlier call* whose cache this call reads instead of keeping one (its mixer then writes
-    nothing); ``None`` = the call keeps its own."""
+    nothing); ``None`` = the call keeps its own.  ``entrance`` = what the stream goes through right before this call
+    (several calls may name the same one, told apart by ``entrance_number``), or None."""
 
     layer: int
     cache_of: Optional[int] = None
+    entrance: Optional[Entrance] = None
+    entrance_number: int = 0
 
 
 @dataclass
@@ -49,9 +52,13 @@ class ModelSpec:
             for sub in part.sub_parts().values():
                 add(sub)
 
-        for part in (self.embedding, *self.layers, self.final_norm, self.lm_head):
+        for part in (self.embedding, *self.entrances(), *self.layers, self.final_norm, self.lm_head):
             add(part)
         return out
+
+    def entrances(self) -> List[Entrance]:
+        """Every entrance that the schedule names, once."""
+        return list({id(c.entrance): c.entrance for c in self.schedule if c.entrance is not None}.values())
 
     def stream_norms(self) -> List[Norm]:
         """The norms that read the residual stream and fold its pending delta in: those a block

@@ -89,17 +89,19 @@ def rmsnorm(residual: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype:
             delta: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None,
             write_back: bool = False, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """RMSNorm of ``residual (+ delta)`` (float32 stream) times ``weight`` (float32).  ``delta``
-    is [T, H] in ``out_dtype``, or float32 [S, T, H] with S in (2, 4, 8): partial sums that are
+    is [T, H] in ``out_dtype`` or in float32, or float32 [S, T, H]: partial sums that are
     added in order.  ``write_back`` stores the sum into ``residual``; ``rows`` (int32) selects rows."""
     _need(residual, "rmsnorm residual", dtype=torch.float32, ndim=2)
     t, h = residual.shape
     _need(weight, "rmsnorm weight", dtype=torch.float32, shape=(h,))
     n_parts = 0
+    if delta is not None and delta.ndim == 2 and delta.dtype == torch.float32 and out_dtype != torch.float32:
+        delta = delta.unsqueeze(0)  # an unrounded delta beside 16-bit activations: one plane of sums
     if delta is not None and delta.ndim == 3:
         n_parts = delta.shape[0]
         _need(delta, "rmsnorm delta parts", dtype=torch.float32, shape=(n_parts, t, h))
-        if not 2 <= n_parts <= GEMM_MAX_SPLITS:
-            raise KernelError(f"rmsnorm: {n_parts} partial sums; 2 to {GEMM_MAX_SPLITS} are taken")
+        if not 1 <= n_parts <= GEMM_MAX_SPLITS:
+            raise KernelError(f"rmsnorm: {n_parts} partial sums; up to {GEMM_MAX_SPLITS} are taken")
     elif delta is not None:
         _need(delta, "rmsnorm delta", dtype=out_dtype, shape=(t, h))
     n_rows = t
@@ -184,8 +186,31 @@ def gate_act_code(act: str) -> int:
         raise KernelError(f"unknown gate activation '{act}' (known: {sorted(GATE_ACTS)})") from None
 
 
-def swiglu(x: torch.Tensor, out: Optional[torch.Tensor] = None, act: str = "silu") -> torch.Tensor:
-    """act(x[:, 0::2]) * x[:, 1::2] for x [T, 2I] (gate and up interleaved); ``act``: "silu" or "gelu_tanh"."""
+class GateAct:
+    """What a gated feed-forward makes of a gate and its up value: the name of a gate activation (``GATE_ACTS``: act(g) u),
+    or "clipped" with its two constants: with g cut off above at ``limit`` and u on both sides, g sigmoid(slope g) (u + 1)."""
+
+    __slots__ = ("code", "limit", "slope")
+
+    def __init__(self, name: str, limit: float = 0.0, slope: float = 0.0):
+        if name == "clipped" and not (limit > 0.0 and slope > 0.0):
+            raise KernelError(f"gate activation 'clipped': limit {limit} and slope {slope} must be positive")
+        self.code = 3 if name == "clipped" else gate_act_code(name)
+        self.limit, self.slope = float(limit), float(slope)
+
+    @property
+    def args(self):
+        return self.code, self.limit, self.slope
+
+
+def gate_act(act) -> GateAct:
+    """``act`` as a ``GateAct`` (it may be one, or the name of one without constants)."""
+    return act if isinstance(act, GateAct) else GateAct(act)
+
+
+def swiglu(x: torch.Tensor, out: Optional[torch.Tensor] = None, act="silu") -> torch.Tensor:
+    """The products of gates x[:, 0::2] and up values x[:, 1::2] (``act``: a ``GateAct`` or its name: act(gate) * up) for
+    x [T, 2I]."""
     _need(x, "swiglu input", ndim=2)
     t, two_i = x.shape
     if two_i % 2:
@@ -194,7 +219,7 @@ def swiglu(x: torch.Tensor, out: Optional[torch.Tensor] = None, act: str = "silu
     if out is None:
         out = torch.empty((t, inter), dtype=x.dtype, device=x.device)
     _need(out, "swiglu out", dtype=x.dtype, shape=(t, inter))
-    check(load().fsie_gated_act(x.data_ptr(), out.data_ptr(), t, inter, dtype_code(x.dtype), gate_act_code(act), _stream()))
+    check(load().fsie_gated_act(x.data_ptr(), out.data_ptr(), t, inter, dtype_code(x.dtype), *gate_act(act).args, _stream()))
     return out
 
 
@@ -421,6 +446,21 @@ def gemm_mfma_skinny(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch
     return out
 
 
+def gemm_mfma_skinny_gated(x: torch.Tensor, weight: torch.Tensor, act, waves: int = 0, blocks: int = 0) -> torch.Tensor:
+    """The products of gate and up value (``act``: a ``GateAct`` or its name) [M, N/2] in bfloat16, gate and up rows of
+    ``weight`` [N, K] in turn, by the few-rows product: up to 16 rows, K a multiple of 8."""
+    _need(x, "gemm x", dtype=torch.bfloat16, ndim=2)
+    _need(weight, "gemm weight", dtype=torch.bfloat16, ndim=2)
+    m, k = x.shape
+    n = weight.shape[0]
+    if weight.shape[1] != k or n % 2:
+        raise KernelError(f"gemm: weight {tuple(weight.shape)} against rows of {k}: gate and up rows in turn are an even number")
+    out = torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
+    check(load().fsie_gemm_mfma_skinny_gated(x.data_ptr(), weight.data_ptr(), out.data_ptr(), m, n, k, waves, blocks,
+                                             *gate_act(act).args, _stream()))
+    return out
+
+
 def gemm_mfma_skinny_act(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], act: PointAct,
                          waves: int = 0, blocks: int = 0) -> torch.Tensor:
     """act(x . weight^T + bias) [M, N] in bfloat16 by the few-rows product, the activation in its epilogue: up to 16 rows,
@@ -498,8 +538,8 @@ def gemm_mfma_wide_splits_ok(k: int, splits: int) -> bool:
 
 
 def gemm_mfma_wide_swiglu(x: torch.Tensor, weight: torch.Tensor, waves: int = 0, blocks: int = 0,
-                          out: Optional[torch.Tensor] = None, act: str = "silu") -> torch.Tensor:
-    """silu(gate) * up [M, N/2] (bfloat16) of x [M, K] and a weight [N, K] whose rows are gate and up
+                          out: Optional[torch.Tensor] = None, act="silu") -> torch.Tensor:
+    """silu(gate) * up, or what ``act`` (a ``GateAct`` or its name) makes of them, [M, N/2] (bfloat16) of x [M, K] and a weight [N, K] whose rows are gate and up
     in turn (or its ``FragmentOrdered`` copy), by the kernel that shares x through LDS; up to 64
     rows, N a multiple of 4, K of 128."""
     _need(x, "gemm x", dtype=torch.bfloat16, ndim=2)
@@ -511,7 +551,7 @@ def gemm_mfma_wide_swiglu(x: torch.Tensor, weight: torch.Tensor, waves: int = 0,
         out = torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
     _need(out, "gemm out", dtype=torch.bfloat16, shape=(m, n // 2))
     check(load().fsie_gemm_mfma_wide_gated(x.data_ptr(), wptr, out.data_ptr(), m, n, k, waves, blocks, frags,
-                                           gate_act_code(act), _stream()))
+                                           *gate_act(act).args, _stream()))
     return out
 
 
@@ -944,6 +984,38 @@ def sandwich_norm(residual: torch.Tensor, delta: torch.Tensor, post_weight: torc
     return out
 
 
+def stream_out(residual: torch.Tensor, delta: Optional[torch.Tensor], post_weight: Optional[torch.Tensor], post_eps: float,
+               out: torch.Tensor, restart: torch.Tensor) -> torch.Tensor:
+    """``out`` [T, H] (columns of wider rows may do) receives the stream, ``residual`` plus what is pending (``delta`` None:
+    nothing; ``post_weight``: delta's RMS norm), rounded to its type; every row of ``residual`` becomes ``restart``
+    (float32 [H]), on which what comes next is a delta.  ``delta`` as for ``sandwich_norm``."""
+    _need(residual, "stream_out residual", dtype=torch.float32, ndim=2)
+    t, h = residual.shape
+    _need(restart, "stream_out restart", dtype=torch.float32, shape=(h,))
+    out = _columns_of(out, t, h, out.dtype, residual.device, "stream_out")
+    n_parts = 0
+    if post_weight is not None:
+        _need(post_weight, "stream_out post weight", dtype=torch.float32, shape=(h,))
+    if delta is not None and delta.ndim == 2 and delta.dtype == torch.float32 and out.dtype != torch.float32:
+        delta = delta.unsqueeze(0)
+    if delta is not None:
+        n_parts = _delta_parts(delta, t, h, out.dtype, "stream_out")
+    elif post_weight is not None:
+        raise KernelError("stream_out: the norm of a delta that is not there")
+    check(load().fsie_stream_out(residual.data_ptr(), _ptr(delta), _ptr(post_weight), float(post_eps), out.data_ptr(),
+                                 out.stride(0) if t else h, restart.data_ptr(), t, h, dtype_code(out.dtype), n_parts, _stream()))
+    return out
+
+
+def round_columns(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """``out`` [T, N] (columns of wider rows may do) = float32 ``x`` [T, N] rounded to its type."""
+    _need(x, "round_columns x", dtype=torch.float32, ndim=2)
+    t, n = x.shape
+    out = _columns_of(out, t, n, out.dtype, x.device, "round_columns")
+    check(load().fsie_round_columns(x.data_ptr(), out.data_ptr(), out.stride(0) if t else n, t, n, dtype_code(out.dtype), _stream()))
+    return out
+
+
 def _columns_of(out: Optional[torch.Tensor], t: int, width: int, dtype, device, name: str) -> torch.Tensor:
     """``out`` (or a new tensor) as the place of a result [t, width]: it may be a run of columns of wider rows."""
     if out is None:
@@ -1049,17 +1121,18 @@ def gla_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, z: torch.Te
 # attention through a latent
 # ---------------------------------------------------------------------------------------------
 def latent_prep(proj: torch.Tensor, dq_off: int, q_rank: int, dkv_off: int, kv_rank: int, rot_dim: int, rot_pairs: int,
-                g_off: int, heads: int, q_weight: torch.Tensor, kv_weight: Optional[torch.Tensor], eps: float,
+                g_off: int, heads: int, q_weight: Optional[torch.Tensor], kv_weight: Optional[torch.Tensor], eps: float,
                 cos_sin: Optional[torch.Tensor], slots: Optional[torch.Tensor] = None,
                 k_pool: Optional[torch.Tensor] = None, v_pool: Optional[torch.Tensor] = None):
-    """From the fused projection ``proj`` [T, W]: the normed query latent [T, q_rank] (type of ``proj``), the
-    sigmoid of the heads' gates (float32 [T, heads]) and, if pools are given, every token's cache row
+    """From the fused projection ``proj`` [T, W]: the normed query latent [T, q_rank] (type of ``proj``; q_rank 0: there is
+    none), the sigmoid of the heads' gates (float32 [T, heads]) and, if pools are given, every token's cache row
     [normed latent | key part with its first ``rot_pairs`` pairs of neighbours rotated (a negative number: that
     many pairs of value i with value i + pairs) | zeros] written at
     ``slots`` into ``k_pool`` [units, 1, page, width] and (transposed) ``v_pool`` [units, 1, width, page]."""
     _need(proj, "latent proj", ndim=2)
     t, w = proj.shape
-    _need(q_weight, "latent q norm weight", dtype=torch.float32, shape=(q_rank,))
+    if q_rank:
+        _need(q_weight, "latent q norm weight", dtype=torch.float32, shape=(q_rank,))
     width = page_size = pool_slots = 0
     if k_pool is not None:
         _need(k_pool, "k_pool", dtype=proj.dtype, ndim=4)
@@ -1075,7 +1148,7 @@ def latent_prep(proj: torch.Tensor, dq_off: int, q_rank: int, dkv_off: int, kv_r
     cq = torch.empty((t, q_rank), dtype=proj.dtype, device=proj.device)
     gate = torch.empty((t, heads), dtype=torch.float32, device=proj.device)
     check(load().fsie_latent_prep(proj.data_ptr(), w, dq_off, q_rank, dkv_off, kv_rank, rot_dim, rot_pairs, g_off, heads,
-                                  q_weight.data_ptr(), _ptr(kv_weight), float(eps), _ptr(cos_sin), cq.data_ptr(),
+                                  _ptr(q_weight), _ptr(kv_weight), float(eps), _ptr(cos_sin), cq.data_ptr(),
                                   gate.data_ptr(), _ptr(slots), _ptr(k_pool), _ptr(v_pool), width, page_size, pool_slots, t,
                                   dtype_code(proj.dtype), _stream()))
     return cq, gate
@@ -1101,10 +1174,15 @@ def rope_pairs(x: torch.Tensor, in_off: int, in_head_stride: int, out: torch.Ten
 
 
 def head_gemm(x: torch.Tensor, x_off: int, x_head_stride: int, weight: torch.Tensor, out: torch.Tensor, out_off: int,
-              out_head_stride: int, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``out[t, h, n] = (sum_k x[t, h, k] weight[h, n, k]) * gate[t, h]``: a matrix of its own for every head.
-    ``x`` [T, W] holds head h's K values from column ``x_off + h * x_head_stride``, ``out`` [T, V] receives its N
-    values from column ``out_off + h * out_head_stride``; ``weight`` [heads, N, K]; ``gate`` float32 [T, heads]."""
+              out_head_stride: int, gate: Optional[torch.Tensor] = None, gate_rows: Optional[torch.Tensor] = None,
+              turn: Optional[tuple] = None) -> torch.Tensor:
+    """``out[t, h, n] = (sum_k x[t, h, k] weight[h, n, k]) * gate[t, h] * sigmoid(gate_rows[t, h N + n])``: a matrix of its
+    own for every head.  ``x`` [T, W] holds head h's K values from column ``x_off + h * x_head_stride``, ``out`` [T, V]
+    receives its N values from column ``out_off + h * out_head_stride``; ``weight`` [heads, N, K]; ``gate`` float32
+    [T, heads] and ``gate_rows`` [T, heads N] of ``x``'s type (columns of wider rows may do) are factors, or None.
+    ``turn`` = (in, out, width, rot_pairs, out_width, cos_sin): beside the product the run of ``width`` values at column
+    ``in`` of every head of ``x`` is turned as by ``rope_pairs`` and written to column ``out`` of the head of ``out``,
+    zeros up to ``out_width``."""
     _need(x, "head_gemm x", ndim=2)
     _need(weight, "head_gemm weight", dtype=x.dtype, ndim=3)
     _need(out, "head_gemm out", dtype=x.dtype, ndim=2)
@@ -1114,9 +1192,16 @@ def head_gemm(x: torch.Tensor, x_off: int, x_head_stride: int, weight: torch.Ten
         raise KernelError("head_gemm: x and out must have a row a token")
     if gate is not None:
         _need(gate, "head_gemm gate", dtype=torch.float32, shape=(t, heads))
+    if gate_rows is not None and (not gate_rows.is_cuda or gate_rows.dtype != x.dtype or gate_rows.stride(1) != 1
+                                  or tuple(gate_rows.shape) != (t, heads * n)):
+        raise KernelError(f"head_gemm gate rows: must be [{t}, {heads * n}] of {x.dtype} on the GPU with contiguous rows")
+    t_in, t_out, t_width, pairs, t_out_width, cos_sin = turn if turn is not None else (0, 0, 0, 0, 0, None)
+    if pairs:
+        _need(cos_sin, "head_gemm cos/sin", dtype=torch.float32, shape=(t, abs(pairs), 2))
     check(load().fsie_head_gemm(x.data_ptr(), x.shape[1], x_off, x_head_stride, weight.data_ptr(), out.data_ptr(),
-                                out.shape[1], out_off, out_head_stride, _ptr(gate), t, heads, n, k, dtype_code(x.dtype),
-                                _stream()))
+                                out.shape[1], out_off, out_head_stride, _ptr(gate), _ptr(gate_rows),
+                                gate_rows.stride(0) if gate_rows is not None and t else heads * n, t_in, t_out, t_width, pairs,
+                                t_out_width, _ptr(cos_sin), t, heads, n, k, dtype_code(x.dtype), _stream()))
     return out
 
 
@@ -1439,12 +1524,12 @@ def moe_group(ids: torch.Tensor, experts: int, tile_rows: Optional[int] = None):
 
 def moe_gemm(a: torch.Tensor, weight: torch.Tensor, tiles: torch.Tensor, order: torch.Tensor, gather_div: int = 0,
              pair_weight: Optional[torch.Tensor] = None, tile_rows: Optional[int] = None,
-             gated: Optional[str] = None) -> torch.Tensor:
+             gated=None) -> torch.Tensor:
     """One product per expert: out[slot] = a[row(slot)] . weight[expert of slot]^T with ``weight`` [E, N, K].
     ``gather_div`` > 0: row(slot) = order[slot] // gather_div (``a`` holds tokens); 0: row(slot) = slot.  Without
     ``pair_weight`` the result is the exact GELU of the product in ``a``'s type; with it (float32 [pairs]) the product
     times the pair's weight, float32.  ``tile_rows``: the rows of a tile of ``tiles`` (default: what ``moe_tile_rows``
-    names for the step, as ``moe_group``'s default is).  ``gated`` (a gate activation's name): the rows of every
+    names for the step, as ``moe_group``'s default is).  ``gated`` (a ``GateAct`` or its name): the rows of every
     expert's matrix are gate and up in turn and the result is act(gate) * up, [slots, N / 2]."""
     _need(a, "moe_gemm a", ndim=2)
     _need(weight, "moe_gemm weight", dtype=a.dtype, ndim=3)
@@ -1463,19 +1548,27 @@ def moe_gemm(a: torch.Tensor, weight: torch.Tensor, tiles: torch.Tensor, order: 
             raise KernelError("moe_gemm: one weight a pair")
     if gated is not None and (pair_weight is not None or n % 2):
         raise KernelError("moe_gemm: a gated product has an even number of rows and no pair weights")
-    epilogue = 2 + gate_act_code(gated) if gated is not None else (1 if pair_weight is not None else 0)
+    pair = gate_act(gated) if gated is not None else None
+    epilogue = 2 + pair.code if pair is not None else (1 if pair_weight is not None else 0)
     out = torch.empty((slots, n // 2 if gated is not None else n), dtype=torch.float32 if pair_weight is not None else a.dtype,
                       device=a.device)
     check(load().fsie_moe_gemm(a.data_ptr(), weight.data_ptr(), out.data_ptr(), tiles.data_ptr(), tiles.shape[0],
                                order.data_ptr(), int(gather_div), _ptr(pair_weight), n, k, epilogue,
-                               dtype_code(a.dtype), tile_rows, _stream()))
+                               dtype_code(a.dtype), tile_rows, *(pair.args[1:] if pair is not None else (0.0, 0.0)), _stream()))
     return out
 
 
-def moe_combine(rows: torch.Tensor, slot_of: torch.Tensor, n_tokens: int, top: int) -> torch.Tensor:
-    """float32 [T, H]: for every token the sum of its ``top`` rows (``rows`` [pairs, H] by slot), in the order of its choices."""
+def moe_combine(rows: torch.Tensor, slot_of: torch.Tensor, n_tokens: int, top: int,
+                shared: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """float32 [T, H]: for every token the sum of its ``top`` rows (``rows`` [pairs, H] by slot), in the order of its choices,
+    plus its row of ``shared``: [T, H] in bfloat16 or float32, or float32 partial sums [S, T, H]."""
+    parts, dtype = 0, torch.float32
+    if shared is not None:
+        dtype = shared.dtype
+        parts = _delta_parts(shared, n_tokens, rows.shape[1], dtype, "moe_combine shared")
     _need(rows, "moe_combine rows", dtype=torch.float32, ndim=2)
     _need(slot_of, "moe_combine slot_of", dtype=torch.int32, shape=(n_tokens * top,))
     y = torch.empty((n_tokens, rows.shape[1]), dtype=torch.float32, device=rows.device)
-    check(load().fsie_moe_combine(rows.data_ptr(), slot_of.data_ptr(), y.data_ptr(), n_tokens, top, rows.shape[1], _stream()))
+    check(load().fsie_moe_combine(rows.data_ptr(), slot_of.data_ptr(), y.data_ptr(), n_tokens, top, rows.shape[1],
+                                  _ptr(shared), parts, dtype_code(dtype), _stream()))
     return y

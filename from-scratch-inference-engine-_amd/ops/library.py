@@ -35,6 +35,7 @@ _SIGNATURES = {
     "fsie_swiglu": ([_P, _P, c_int, c_int, c_int, _P], c_int),
     "fsie_residual_add": ([_P, _P, c_int64, c_int, _P], c_int),
     "fsie_round_to": ([_P, _P, c_int64, c_int, _P], c_int),
+    "fsie_round_columns": ([_P, _P, c_int64, c_int, c_int, c_int, _P], c_int),
     "fsie_scaled_sum": ([_P, c_float, _P, c_float, _P, c_int64, c_int, _P], c_int),
     "fsie_pool_blocks": ([_P, _P, _P, c_int, c_int, _P, _P, _P, c_int, c_int, _P, c_int, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_bias_add": ([_P, _P, c_int, c_int, c_int, _P], c_int),
@@ -78,8 +79,10 @@ _SIGNATURES = {
     "fsie_static_scratch_bytes": ([], c_int64),
     "fsie_attention_split_static": ([_P, c_int64, _P, _P, _P, c_int, _P, c_int, _P, c_int, c_int, _P, c_int, c_int,
                                      c_int, c_int, c_int, c_float, c_int, c_int, c_int, _P], c_int),
-    "fsie_gated_act": ([_P, _P, c_int, c_int, c_int, c_int, _P], c_int),
-    "fsie_gemm_mfma_wide_gated": ([_P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P], c_int),
+    "fsie_gated_act": ([_P, _P, c_int, c_int, c_int, c_int, c_float, c_float, _P], c_int),
+    "fsie_gemm_mfma_wide_gated": ([_P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, _P], c_int),
+    "fsie_gemm_mfma_skinny_gated": ([_P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, _P], c_int),
+    "fsie_stream_out": ([_P, _P, _P, c_float, _P, c_int64, _P, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_sandwich_norm": ([_P, _P, _P, _P, c_float, _P, c_float, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_gated_headnorm": ([_P, c_int, _P, c_int64, _P, _P, c_int, c_int, c_int, c_float, c_int, c_int, c_int64, c_float, _P], c_int),
     "fsie_gla_scan_shape": ([c_int, c_int, c_int, ctypes.POINTER(c_int), ctypes.POINTER(c_int), ctypes.POINTER(c_int),
@@ -91,8 +94,8 @@ _SIGNATURES = {
                           _P, _P, _P, c_int, c_int, c_int64, c_int, c_int, _P], c_int),
     "fsie_rope_pairs": ([_P, c_int64, c_int, c_int, _P, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, _P, c_int, c_int,
                          _P], c_int),
-    "fsie_head_gemm": ([_P, c_int64, c_int, c_int, _P, _P, c_int64, c_int, c_int, _P, c_int, c_int, c_int, c_int, c_int, _P],
-                       c_int),
+    "fsie_head_gemm": ([_P, c_int64, c_int, c_int, _P, _P, c_int64, c_int, c_int, _P, _P, c_int64, c_int, c_int, c_int, c_int,
+                        c_int, _P, c_int, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_rope_table_scaled": ([_P, _P, c_int, c_int, c_float, _P, _P], c_int),
     "fsie_layer_norm": ([_P, _P, c_int, _P, c_int, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_float, c_int, c_int, c_int, _P],
                         c_int),
@@ -113,9 +116,9 @@ _SIGNATURES = {
     "fsie_mlstm_out": ([_P, _P, _P, _P, c_int64, _P, _P, c_int, c_int, c_int, c_float, c_int, _P], c_int),
     "fsie_moe_route": ([_P, _P, _P, c_int, _P, _P, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_int, _P], c_int),
     "fsie_moe_group": ([_P, c_int, c_int, c_int, _P, _P, _P, c_int, _P], c_int),
-    "fsie_moe_gemm": ([_P, _P, _P, _P, c_int, _P, c_int, _P, c_int, c_int, c_int, c_int, c_int, _P], c_int),
+    "fsie_moe_gemm": ([_P, _P, _P, _P, c_int, _P, c_int, _P, c_int, c_int, c_int, c_int, c_int, c_float, c_float, _P], c_int),
     "fsie_moe_tile_rows": ([c_int, c_int], c_int),
-    "fsie_moe_combine": ([_P, _P, _P, c_int, c_int, c_int, _P], c_int),
+    "fsie_moe_combine": ([_P, _P, _P, c_int, c_int, c_int, _P, c_int, c_int, _P], c_int),
     "fsie_sample": ([_P, c_int, c_int, _P, _P, _P, _P, _P, _P], c_int),
 }
 

@@ -19,6 +19,7 @@ Kinds and their interfaces (``ctx`` is the step's ``StepContext``):
                    in place by the step's positions.  It touches nothing else: bias, norms of q
                    and k and the write into the cache are the mixer's.
   Block            the arrangement: ``block.forward(hidden, ctx, cache)``.
+  Entrance         what stands before a call of the model's schedule: ``entrance.forward(hidden, ctx, number)``.
 """
 
 from __future__ import annotations
@@ -210,9 +211,23 @@ class Block(Part):
         raise NotImplementedError
 
 
+class Entrance(Part):
+    """What the stream goes through before a call of the model's schedule (``LayerCall.entrance``): a map of the whole
+    stream that belongs to no layer, such as what stands before every pass of layers that run several times."""
+
+    kind = "entrance"
+
+    def begin(self, hidden: HiddenState, ctx) -> None:
+        """Called once a forward pass, when ``hidden`` is the embedding's output: for an entrance that reads it later."""
+
+    def forward(self, hidden: HiddenState, ctx, number: int) -> None:
+        """Replaces the stream; ``number`` is the call's ``LayerCall.entrance_number``."""
+        raise NotImplementedError
+
+
 # ------------------------------------------------------------------------------ registries
 _REGISTRIES: Dict[str, Dict[str, Callable[..., Part]]] = {
-    "norm": {}, "mixer": {}, "feed_forward": {}, "position": {}, "block": {}, "convolution": {},
+    "norm": {}, "mixer": {}, "feed_forward": {}, "position": {}, "block": {}, "convolution": {}, "entrance": {},
 }
 
 

@@ -132,6 +132,16 @@ class Linear:
         long inner dimension the matrix-core kernel cuts K into slices with workgroups of their
         own, which fills the chip where N alone leaves too few of them, and returns their float32
         partial sums [S, T, N]; the next norm adds them up in order."""
+        sums = self.residual_sums(x, ctx)
+        return self(x) if sums is None else sums
+
+    def for_stream(self, x: torch.Tensor, ctx) -> torch.Tensor:
+        """The same for a delta that is the whole stream: never rounded to 16 bits (partial sums, or [T, N] in float32)."""
+        sums = self.residual_sums(x, ctx)
+        return self(x, out_dtype=torch.float32) if sums is None else sums
+
+    def residual_sums(self, x: torch.Tensor, ctx) -> Optional[torch.Tensor]:
+        """The partial sums of ``for_residual``, or None where the product is better left whole."""
         m = x.shape[0]
         if (getattr(ctx, "partial_sums_ok", False) and x.dtype == torch.bfloat16 and self.bias is None
                 and GEMM_MFMA_SKINNY_MAX_M < m <= GEMM_MFMA_WIDE_MAX_M and self.streamed is not None):
@@ -150,7 +160,7 @@ class Linear:
             splits = self.residual_splits(m)
             if splits > 1:
                 return ops.gemm_mfma_skinny(x, self.weight, splits=splits)
-        return self(x)
+        return None
 
     def partial_sums(self, x: torch.Tensor, few_rows: bool = False) -> Optional[torch.Tensor]:
         """x . W^T (no bias) of 17 to 64 rows (to 128 from a fragment-ordered copy) as float32 partial
