@@ -319,15 +319,35 @@ def romepel_shape(width: int, ff: int, layers: int, vocab: int) -> dict:
             "logit_softcap": 30.0, "layers": out}
 
 
+def nenizen_shape(width: int, ff: int, layers: int, vocab: int) -> dict:
+    """A Nenizen configuration of real layer sizes: six layers of which the second to fourth run twice (so ``layers`` = 9 of
+    them run), attention through latents of 192 + 64 values of each of the three kinds (the windowed one over 1,024
+    positions), dense feed-forwards and eight routed experts beside a shared one in turn (an expert has ff / 8, two a token)."""
+    heads = width // 128
+    latent = {"heads": heads, "dim": 64, "rot_dim": 64, "vdim": 128, "kv_rank": 192, "scale": 128 ** -0.5,
+              "rot": {"base": 500000.0, "dims": 64}}
+    kinds = {"latent_attention": latent, "latent_attention_2": {**latent, "q_rank": width // 2 + 256, "mask": {"size": 1024}},
+             "latent_attention_3": {**latent, "q_rank": width // 2 + 256}}
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    routed = {"kind": "moe", "expert": {"ff": ff // 8}, "router": {"experts": 8, "top": 2}, "shared": {"ff": ff // 8}}
+    order = ("_3", "", "_2", "", "_3", "")
+    if layers != 9:
+        raise ValueError("the looped shape is made for nine runs of layers")
+    return {"architecture": "Nenizen", "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "embedding": {"scale": 4.0},
+            "logit_softcap": 30.0, "loop": {"start": 1, "stop": 4, "times": 2},
+            "layers": [{"type": "latent_attention" + k, "mixer": dict(kinds["latent_attention" + k]),
+                        "mlp": dict(routed if k == "" else dense)} for k in order]}
+
+
 DESIGN_SHAPES = {"gilozen": gilozen_shape, "botulorn": botulorn_shape, "fiterax": fiterax_shape, "mafosun": mafosun_shape,
-                 "romepel": romepel_shape}
+                 "romepel": romepel_shape, "nenizen": nenizen_shape}
 # a design whose mechanisms an earlier one shares is measured beside that one too
-DESIGN_BESIDE = {"romepel": ("gilozen",)}
+DESIGN_BESIDE = {"romepel": ("gilozen",), "nenizen": ("gilozen", "mafosun")}
 DESIGN_SIZES = {"2048": (2048, 8192, 9, 32000), "4096": (4096, 14336, 9, 32000)}  # width, ff, layers, vocab
 
 
 def design_comparison(args) -> int:
-    """--workload gilozen | botulorn | fiterax | mafosun | romepel: prefill (one prompt of 2,048 tokens in one step) and decode (batches of 8 and 64 at a
+    """--workload gilozen | botulorn | fiterax | mafosun | romepel | nenizen: prefill (one prompt of 2,048 tokens in one step) and decode (batches of 8 and 64 at a
     context of 512, from captured graphs) of the named design at two real layer sizes with random weights, beside a Qwen2
     model of the same width, feed-forward, layers and vocabulary (grouped-query attention, 128 values a head, four
     query heads a key/value head) through the same step function.  One JSON line."""
@@ -415,15 +435,15 @@ def main() -> int:
     ap.add_argument("--no-tune", action="store_true", help="leave the library's kernel choice for prefill to its heuristic")
     ap.add_argument("--no-streamed-copies", action="store_true",
                     help="do not keep the large weights a second time in the order of the matrix instruction's fragments")
-    ap.add_argument("--design-sizes", default="2048,4096", help="--workload gilozen | botulorn | fiterax | mafosun | romepel: widths to run (2048, 4096)")
-    ap.add_argument("--design-batches", default="8,64", help="--workload gilozen | botulorn | fiterax | mafosun | romepel: decode batches to time (at most 64)")
-    ap.add_argument("--design-phases", default="prefill,decode", help="--workload gilozen | botulorn | fiterax | mafosun | romepel: what to time (for a trace of one phase)")
-    ap.add_argument("--design-models", default="", help="--workload gilozen | botulorn | fiterax | mafosun | romepel: of the models compared, only these (for a trace of one)")
-    ap.add_argument("--workload", choices=["decode", "mixed", "long-prefill", "gilozen", "botulorn", "fiterax", "mafosun", "romepel"], default="decode",
+    ap.add_argument("--design-sizes", default="2048,4096", help="--workload gilozen | botulorn | fiterax | mafosun | romepel | nenizen: widths to run (2048, 4096)")
+    ap.add_argument("--design-batches", default="8,64", help="--workload gilozen | botulorn | fiterax | mafosun | romepel | nenizen: decode batches to time (at most 64)")
+    ap.add_argument("--design-phases", default="prefill,decode", help="--workload gilozen | botulorn | fiterax | mafosun | romepel | nenizen: what to time (for a trace of one phase)")
+    ap.add_argument("--design-models", default="", help="--workload gilozen | botulorn | fiterax | mafosun | romepel | nenizen: of the models compared, only these (for a trace of one)")
+    ap.add_argument("--workload", choices=["decode", "mixed", "long-prefill", "gilozen", "botulorn", "fiterax", "mafosun", "romepel", "nenizen"], default="decode",
                     help="decode: the default run.  mixed: --requests prompts of --min-prompt to --max-prompt tokens, "
                          "--outputs tokens each, through the scheduler (made for --shape 14b).  "
                          "long-prefill: one prompt of --prefill-tokens tokens in portions of the token budget "
-                         "(made for --shape 32b).  gilozen, botulorn, fiterax, mafosun, romepel: that design beside Qwen2 at equal layer sizes")
+                         "(made for --shape 32b).  gilozen, botulorn, fiterax, mafosun, romepel, nenizen: that design beside Qwen2 at equal layer sizes")
     ap.add_argument("--requests", type=int, default=32)
     ap.add_argument("--min-prompt", type=int, default=128)
     ap.add_argument("--max-prompt", type=int, default=4096)

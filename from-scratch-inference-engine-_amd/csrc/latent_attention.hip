@@ -117,6 +117,7 @@ template <typename T>
 __device__ __forceinline__ void turn_heads(const HeadExtras<T>& ex, const T* __restrict__ x, int64_t x_stride, int x_first,
                                            T* __restrict__ y, int64_t y_stride, int y_first, int t0, int tokens) {
     const int n = ex.rot_pairs < 0 ? -ex.rot_pairs : ex.rot_pairs;
+#pragma unroll 4
     for (int e = threadIdx.x; e < tokens * ex.rot_out_width; e += kThreads) {
         const int i = e / ex.rot_out_width, j = e - i * ex.rot_out_width;
         const int64_t t = t0 + i;
@@ -193,8 +194,9 @@ __global__ __launch_bounds__(kThreads) void head_gemm_kernel(const T* __restrict
 // The same product on the matrix cores, bfloat16 operands and float32 sums (v_mfma_f32_16x16x32_bf16): both x's
 // and w's rows run along K, which is what the instruction's operands want of a lane (eight neighbouring K
 // values of one row), so both are read from memory as they lie, no staging.  w is the first operand: a lane
-// then ends with four neighbouring outputs of one token, one 8-byte store.  A wave computes MT tiles of
-// sixteen tokens by four tiles of sixteen outputs; the four waves of a workgroup are next to each other along N.
+// then ends with four neighbouring outputs of one token, one 8-byte store (where the rows allow it: `wide`).  A wave
+// computes MT tiles of sixteen tokens by four tiles of sixteen outputs; WN of the four waves of a workgroup are next to each
+// other along N, the others along the tokens.
 // Rows must start at multiples of eight values (16 bytes) and K must be one.
 typedef __bf16 hg_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float hg_floatx4 __attribute__((ext_vector_type(4)));
@@ -204,18 +206,21 @@ union HgFrag {
     hg_bf16x8 v;
 };
 
-template <int MT>
+template <int MT, int WN>
 __global__ __launch_bounds__(kThreads) void head_gemm_mfma_kernel(const bf16_t* __restrict__ x, int64_t x_stride, int x_off,
                                                                   int x_hs, const bf16_t* __restrict__ w,
                                                                   bf16_t* __restrict__ y, int64_t y_stride, int y_off,
                                                                   int y_hs, HeadExtras<bf16_t> ex, int n_tokens,
-                                                                  int heads, int N, int K) {
+                                                                  int heads, int N, int K, int wide) {
     const int h = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const int n0 = (blockIdx.x * 4 + wave) * 64, t0 = blockIdx.y * (16 * MT);
+    constexpr int kTokens = 16 * MT * (4 / WN);  // of a workgroup
     if (ex.rot_out_width && blockIdx.x == gridDim.x - 1) {
-        turn_heads(ex, x, x_stride, x_off + h * x_hs, y, y_stride, y_off + h * y_hs, t0, min(16 * MT, n_tokens - t0));
+        const int first = blockIdx.y * kTokens;
+        turn_heads(ex, x, x_stride, x_off + h * x_hs, y, y_stride, y_off + h * y_hs, first, min(kTokens, n_tokens - first));
         return;
     }
+    const int n0 = (blockIdx.x * WN + wave % WN) * 64, t0 = blockIdx.y * kTokens + wave / WN * (16 * MT);
+    if (t0 >= n_tokens) return;
     if (n0 >= N) return;
     const int r = lane & 15, kq = (lane >> 4) * 8;
     const bf16_t* wh = w + static_cast<int64_t>(h) * N * K;
@@ -242,6 +247,7 @@ __global__ __launch_bounds__(kThreads) void head_gemm_mfma_kernel(const bf16_t* 
         for (int b = 0; b < MT; ++b) acc[a][b] = hg_floatx4{0.f, 0.f, 0.f, 0.f};
     }
     const hg_u32x4 zero = {0u, 0u, 0u, 0u};
+#pragma unroll 2
     for (int k0 = 0; k0 < K; k0 += 32) {
         const bool kok = k0 + kq < K;  // K is a multiple of eight: a lane's eight values are all inside or all outside
         HgFrag wf[4], xf[MT];
@@ -265,6 +271,24 @@ __global__ __launch_bounds__(kThreads) void head_gemm_mfma_kernel(const bf16_t* 
 #pragma unroll
         for (int a = 0; a < 4; ++a) {
             const int n = n0 + 16 * a + nq;
+            if (wide) {  // (N is a multiple of four: all four outputs are there or none)
+                if (n >= N) continue;
+                float g[4];
+                const float head_gate = ex.gate ? ex.gate[static_cast<int64_t>(t) * heads + h] : 1.0f;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) g[i] = head_gate;
+                if (ex.gate_rows) {
+                    const uint2 z = *reinterpret_cast<const uint2*>(ex.gate_rows + static_cast<int64_t>(t) * ex.gate_stride +
+                                                                    static_cast<int64_t>(h) * N + n);
+                    const float zs[4] = {__uint_as_float(z.x << 16), __uint_as_float(z.x & 0xffff0000u),
+                                         __uint_as_float(z.y << 16), __uint_as_float(z.y & 0xffff0000u)};
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) g[i] *= 1.0f / (1.0f + expf(-zs[i]));
+                }
+                *reinterpret_cast<uint2*>(dst + n) = uint2{pack2_bf16(acc[a][b][0] * g[0], acc[a][b][1] * g[1]),
+                                                           pack2_bf16(acc[a][b][2] * g[2], acc[a][b][3] * g[3])};
+                continue;
+            }
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 if (n + i < N)
@@ -362,20 +386,25 @@ extern "C" int fsie_head_gemm(const void* x, int64_t x_stride, int x_off, int x_
     const bool aligned = K % 8 == 0 && x_stride % 8 == 0 && x_off % 8 == 0 && x_hs % 8 == 0 &&
                          reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0;
     if (dtype == FSIE_BF16 && aligned) {
-        const bool two = n_tokens > 16;
-        const int token_tiles = (n_tokens + (two ? 32 : 16) - 1) / (two ? 32 : 16);
+        // whole 8-byte stores (and loads of the gates' logits): every run of four outputs starts at a multiple of 8 bytes
+        const int wide = N % 4 == 0 && y_stride % 4 == 0 && y_off % 4 == 0 && y_hs % 4 == 0 && reinterpret_cast<uintptr_t>(y) % 8 == 0 &&
+                         (!gate_rows || (gate_stride % 4 == 0 && reinterpret_cast<uintptr_t>(gate_rows) % 8 == 0));
+        // waves along N only as far as N fills them; few tokens: all of them
+        const int wn = n_tokens <= 16 || N > 128 ? 4 : N > 64 ? 2 : 1;
+        const int wg_tokens = n_tokens <= 16 ? 16 : 32 * (4 / wn);
+        const int token_tiles = (n_tokens + wg_tokens - 1) / wg_tokens;
         FSIE_REQUIRE(token_tiles <= 65535, "head_gemm: %d tokens are more than one launch takes", n_tokens);
-        const dim3 mgrid((N + 255) / 256 + turned, token_tiles, heads);
+        const dim3 mgrid((N + 64 * wn - 1) / (64 * wn) + turned, token_tiles, heads);
         const HeadExtras<bf16_t> ex{gate, static_cast<const bf16_t*>(gate_rows), gate_stride, cs, rot_in, rot_out, rot_width, rot_pairs, rot_out_width};
-        if (two) {
-            head_gemm_mfma_kernel<2><<<mgrid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), x_stride, x_off, x_hs,
-                                                                    static_cast<const bf16_t*>(w), static_cast<bf16_t*>(y),
-                                                                    y_stride, y_off, y_hs, ex, n_tokens, heads, N, K);
-        } else {
-            head_gemm_mfma_kernel<1><<<mgrid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), x_stride, x_off, x_hs,
-                                                                    static_cast<const bf16_t*>(w), static_cast<bf16_t*>(y),
-                                                                    y_stride, y_off, y_hs, ex, n_tokens, heads, N, K);
-        }
+#define FSIE_HEAD_GEMM(MT, WN)                                                                                              \
+    head_gemm_mfma_kernel<MT, WN><<<mgrid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), x_stride, x_off, x_hs,       \
+                                                                static_cast<const bf16_t*>(w), static_cast<bf16_t*>(y),     \
+                                                                y_stride, y_off, y_hs, ex, n_tokens, heads, N, K, wide)
+        if (n_tokens <= 16) FSIE_HEAD_GEMM(1, 4);
+        else if (wn == 4) FSIE_HEAD_GEMM(2, 4);
+        else if (wn == 2) FSIE_HEAD_GEMM(2, 2);
+        else FSIE_HEAD_GEMM(2, 1);
+#undef FSIE_HEAD_GEMM
     } else if (dtype == FSIE_F32) {
         const HeadExtras<float> ex{gate, static_cast<const float*>(gate_rows), gate_stride, cs, rot_in, rot_out, rot_width, rot_pairs, rot_out_width};
         head_gemm_kernel<float><<<grid, kThreads, 0, stream>>>(static_cast<const float*>(x), x_stride, x_off, x_hs,

@@ -12,15 +12,15 @@ constexpr int kThreads = 256;
 // One block per output row r; source row = rows ? rows[r] : r.
 //   y = delta[row] (+ delta_bias)           (one array of T, or the sum in order of n_parts float32 arrays)
 //   d = y * rsqrt(mean(y^2) + post_eps) * post_weight
-//   v = residual[row] + d;                  if write_back: residual[row] = v
-//   out[r] = v * rsqrt(mean(v^2) + eps) * weight
+//   v = residual[row] + d;                  if write_back: residual[row] = v (restart, if given: restart[0 .. hidden))
+//   out[r] = v * rsqrt(mean(v^2) + eps) * weight   (no weight: v itself; rows of out lie out_stride values apart)
 // The row is kept in LDS between the passes (hidden floats).
 template <typename T>
 __global__ __launch_bounds__(kThreads) void sandwich_norm_kernel(
     float* __restrict__ residual, const T* __restrict__ delta, const float* __restrict__ delta_bias,
     const float* __restrict__ post_weight, float post_eps,
     const float* __restrict__ weight, float eps, T* __restrict__ out, const int32_t* __restrict__ rows, int hidden,
-    int write_back, int n_parts, int64_t part_stride) {
+    int write_back, int n_parts, int64_t part_stride, int64_t out_stride, const float* __restrict__ restart) {
     extern __shared__ float row_buf[];
     __shared__ float scratch[16];
     const int r = blockIdx.x;
@@ -46,11 +46,11 @@ __global__ __launch_bounds__(kThreads) void sandwich_norm_kernel(
     for (int j = threadIdx.x; j < hidden; j += kThreads) {
         const float v = res[j] + (row_buf[j] * post_scale) * post_weight[j];
         row_buf[j] = v;
-        if (write_back) res[j] = v;
+        if (write_back) res[j] = restart ? restart[j] : v;
         sum_sq += v * v;
     }
     const float scale = 1.0f / sqrtf(block_sum(sum_sq, scratch) / static_cast<float>(hidden) + eps);
-    T* dst = out + static_cast<int64_t>(r) * hidden;
+    T* dst = out + static_cast<int64_t>(r) * out_stride;
     for (int j = threadIdx.x; j < hidden; j += kThreads)
         dst[j] = from_float<T>(weight ? (row_buf[j] * scale) * weight[j] : row_buf[j]);  // (no weight: the stream itself)
 }
@@ -78,7 +78,7 @@ __global__ __launch_bounds__(THREADS) void sandwich_norm_vec_kernel(
     float* __restrict__ residual, const T* __restrict__ delta, const float* __restrict__ delta_bias,
     const float* __restrict__ post_weight, float post_eps,
     const float* __restrict__ weight, float eps, T* __restrict__ out, const int32_t* __restrict__ rows, int hidden,
-    int write_back, int n_parts, int64_t part_stride) {
+    int write_back, int n_parts, int64_t part_stride, int64_t out_stride, const float* __restrict__ restart) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
     const int64_t row = rows ? rows[r] : r;
@@ -123,13 +123,13 @@ __global__ __launch_bounds__(THREADS) void sandwich_norm_vec_kernel(
         v[it].z += (y[it].z * post_scale) * wp[it].z;
         v[it].w += (y[it].w * post_scale) * wp[it].w;
         if (j < hidden) {
-            if (write_back) store4(res + j, v[it]);
+            if (write_back) store4(res + j, restart ? load4(restart + j) : v[it]);
             sum_sq += v[it].x * v[it].x + v[it].y * v[it].y + v[it].z * v[it].z + v[it].w * v[it].w;
         }
     }
     // without a weight the stream itself is the result (a layer whose sublayers read the stream as it is)
     const float scale = weight ? 1.0f / sqrtf(block_sum(sum_sq, scratch) / static_cast<float>(hidden) + eps) : 1.f;
-    T* dst = out + static_cast<int64_t>(r) * hidden;
+    T* dst = out + static_cast<int64_t>(r) * out_stride;
 #pragma unroll
     for (int it = 0; it < ITERS; ++it) {
         const int j = (it * THREADS + static_cast<int>(threadIdx.x)) * 4;
@@ -139,37 +139,27 @@ __global__ __launch_bounds__(THREADS) void sandwich_norm_vec_kernel(
     }
 }
 
-// One workgroup a row.  v = residual[row] + what is pending: nothing (delta null), y itself (post_weight null) or the RMS
-// norm of y, with y = delta[row] (one array of T, or the sum in order of n_parts float32 arrays).
-//   out[row][0 .. hidden) = v rounded to T (rows out_stride values apart);  residual[row] = restart[0 .. hidden)
-// The stream goes out and starts again from `restart`: what comes next is a delta on that.
+// The same hand-over of the stream without a norm: one workgroup a row, v = residual[row] + delta[row] (none, one array
+// of T, or the sum in order of n_parts float32 arrays), out[row] = v rounded to T, residual[row] = restart.
 template <typename T>
 __global__ __launch_bounds__(kThreads) void stream_out_kernel(float* __restrict__ residual, const T* __restrict__ delta,
-                                                              const float* __restrict__ post_weight, float post_eps,
                                                               T* __restrict__ out, int64_t out_stride,
                                                               const float* __restrict__ restart, int hidden, int n_parts,
                                                               int64_t part_stride) {
-    extern __shared__ float row_buf[];
-    __shared__ float scratch[16];
     const int64_t row = blockIdx.x;
     float* res = residual + row * hidden;
     const float* parts = n_parts ? reinterpret_cast<const float*>(delta) + row * hidden : nullptr;
     T* dst = out + row * out_stride;
-    float post_scale = 1.f;
-    if (delta) {
-        float sum_sq = 0.f;
-        for (int j = threadIdx.x; j < hidden; j += kThreads) {  // (a thread reads back only what it wrote itself)
-            float y = parts ? parts[j] : to_float(delta[row * hidden + j]);
-#pragma unroll 4
-            for (int s = 1; s < n_parts; ++s) y += parts[s * part_stride + j];
-            row_buf[j] = y;
-            sum_sq += y * y;
-        }
-        if (post_weight) post_scale = 1.0f / sqrtf(block_sum(sum_sq, scratch) / static_cast<float>(hidden) + post_eps);
-    }
     for (int j = threadIdx.x; j < hidden; j += kThreads) {
         float v = res[j];
-        if (delta) v += post_weight ? (row_buf[j] * post_scale) * post_weight[j] : row_buf[j];
+        if (parts) {
+            float y = parts[j];
+#pragma unroll 4
+            for (int s = 1; s < n_parts; ++s) y += parts[s * part_stride + j];
+            v += y;
+        } else if (delta) {
+            v += to_float(delta[row * hidden + j]);
+        }
         dst[j] = from_float<T>(v);
         res[j] = restart[j];
     }
@@ -220,9 +210,10 @@ __global__ void softcap_kernel(float* __restrict__ x, int64_t n, float cap, floa
 // delta: [total_rows][hidden] of the activations' type, or with n_parts > 0 that many float32 arrays
 // [total_rows][hidden] one after the other.  rows (or null): the n_rows source rows to work on.
 // delta_bias [hidden] (or null) is added to every row of it.
-extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const float* delta_bias, const float* post_weight,
-                                  float post_eps, const float* weight, float eps, void* out, const int32_t* rows, int n_rows,
-                                  int hidden, int dtype, int write_back, int n_parts, int total_rows, hipStream_t stream) {
+static int sandwich_norm(float* residual, const void* delta, const float* delta_bias, const float* post_weight,
+                         float post_eps, const float* weight, float eps, void* out, int64_t out_stride, const float* restart,
+                         const int32_t* rows, int n_rows, int hidden, int dtype, int write_back, int n_parts, int total_rows,
+                         hipStream_t stream) {
     FSIE_REQUIRE(n_rows >= 0 && hidden > 0 && hidden <= 16384, "sandwich_norm: bad sizes rows=%d hidden=%d (at most 16384)",
                  n_rows, hidden);
     FSIE_REQUIRE(dtype == FSIE_F32 || dtype == FSIE_BF16, "sandwich_norm: unknown dtype %d", dtype);
@@ -235,14 +226,15 @@ extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const floa
     const bool aligned = hidden % 4 == 0 && reinterpret_cast<uintptr_t>(residual) % 16 == 0 &&
                          reinterpret_cast<uintptr_t>(delta) % 16 == 0 && reinterpret_cast<uintptr_t>(post_weight) % 16 == 0 &&
                          reinterpret_cast<uintptr_t>(delta_bias) % 16 == 0 &&
-                         reinterpret_cast<uintptr_t>(weight) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
+                         reinterpret_cast<uintptr_t>(weight) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0 &&
+                         out_stride % 4 == 0 && reinterpret_cast<uintptr_t>(restart) % 16 == 0;
     if (aligned && hidden <= 8192) {
 #define FSIE_SANDWICH(T, ITERS, THREADS)                                                                             \
     if (delta_bias) FSIE_SANDWICH_WITH(T, ITERS, THREADS, true); else FSIE_SANDWICH_WITH(T, ITERS, THREADS, false)
 #define FSIE_SANDWICH_WITH(T, ITERS, THREADS, BIAS)                                                                  \
     sandwich_norm_vec_kernel<T, ITERS, THREADS, BIAS><<<n_rows, THREADS, 0, stream>>>(                                     \
         residual, static_cast<const T*>(delta), delta_bias, post_weight, post_eps, weight, eps, static_cast<T*>(out), rows, hidden, \
-        write_back, n_parts, part_stride)
+        write_back, n_parts, part_stride, out_stride, restart)
 #define FSIE_SANDWICH_BY_SIZE(T)                                                      \
     if (n_rows <= 128 && hidden > 1024) {  /* few rows: more waves a row */           \
         if (hidden <= 4096) { FSIE_SANDWICH(T, 1, 1024); } else { FSIE_SANDWICH(T, 2, 1024); } \
@@ -265,16 +257,24 @@ extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const floa
     if (dtype == FSIE_F32) {
         sandwich_norm_kernel<float><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const float*>(delta), delta_bias, post_weight,
                                                                      post_eps, weight, eps, static_cast<float*>(out), rows,
-                                                                     hidden, write_back, n_parts, part_stride);
+                                                                     hidden, write_back, n_parts, part_stride, out_stride, restart);
     } else {
         sandwich_norm_kernel<bf16_t><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const bf16_t*>(delta), delta_bias, post_weight,
                                                                       post_eps, weight, eps, static_cast<bf16_t*>(out), rows,
-                                                                      hidden, write_back, n_parts, part_stride);
+                                                                      hidden, write_back, n_parts, part_stride, out_stride, restart);
     }
     FSIE_CHECK_LAUNCH("sandwich_norm");
     return 0;
 }
 
+extern "C" int fsie_sandwich_norm(float* residual, const void* delta, const float* delta_bias, const float* post_weight,
+                                  float post_eps, const float* weight, float eps, void* out, const int32_t* rows, int n_rows,
+                                  int hidden, int dtype, int write_back, int n_parts, int total_rows, hipStream_t stream) {
+    return sandwich_norm(residual, delta, delta_bias, post_weight, post_eps, weight, eps, out, hidden, nullptr, rows, n_rows, hidden,
+                         dtype, write_back, n_parts, total_rows, stream);
+}
+
+// The stream goes out and starts again from `restart`: what comes next is a delta on that.
 extern "C" int fsie_stream_out(float* residual, const void* delta, const float* post_weight, float post_eps, void* out,
                                int64_t out_stride, const float* restart, int n_rows, int hidden, int dtype, int n_parts,
                                hipStream_t stream) {
@@ -283,14 +283,16 @@ extern "C" int fsie_stream_out(float* residual, const void* delta, const float* 
     FSIE_REQUIRE(residual && out && restart && out_stride >= hidden, "stream_out: missing operand");
     FSIE_REQUIRE(n_parts >= 0 && n_parts <= FSIE_GEMM_MAX_SPLITS && (delta || (!n_parts && !post_weight)),
                  "stream_out: %d partial sums, or a norm or sums of nothing", n_parts);
+    if (post_weight)
+        return sandwich_norm(residual, delta, nullptr, post_weight, post_eps, nullptr, 0.f, out, out_stride, restart, nullptr, n_rows,
+                             hidden, dtype, 1, n_parts, n_rows, stream);
     if (n_rows == 0) return 0;
-    const size_t lds = delta ? sizeof(float) * hidden : 0;
     const int64_t part_stride = static_cast<int64_t>(n_rows) * hidden;
     if (dtype == FSIE_F32)
-        stream_out_kernel<float><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const float*>(delta), post_weight, post_eps,
+        stream_out_kernel<float><<<n_rows, kThreads, 0, stream>>>(residual, static_cast<const float*>(delta),
                                                                     static_cast<float*>(out), out_stride, restart, hidden, n_parts, part_stride);
     else
-        stream_out_kernel<bf16_t><<<n_rows, kThreads, lds, stream>>>(residual, static_cast<const bf16_t*>(delta), post_weight, post_eps,
+        stream_out_kernel<bf16_t><<<n_rows, kThreads, 0, stream>>>(residual, static_cast<const bf16_t*>(delta),
                                                                      static_cast<bf16_t*>(out), out_stride, restart, hidden, n_parts, part_stride);
     FSIE_CHECK_LAUNCH("stream_out");
     return 0;
