@@ -389,9 +389,11 @@ extern "C" int fsie_head_gemm(const void* x, int64_t x_stride, int x_off, int x_
         // whole 8-byte stores (and loads of the gates' logits): every run of four outputs starts at a multiple of 8 bytes
         const int wide = N % 4 == 0 && y_stride % 4 == 0 && y_off % 4 == 0 && y_hs % 4 == 0 && reinterpret_cast<uintptr_t>(y) % 8 == 0 &&
                          (!gate_rows || (gate_stride % 4 == 0 && reinterpret_cast<uintptr_t>(gate_rows) % 8 == 0));
-        // waves along N only as far as N fills them; few tokens: all of them
-        const int wn = n_tokens <= 16 || N > 128 ? 4 : N > 64 ? 2 : 1;
-        const int wg_tokens = n_tokens <= 16 ? 16 : 32 * (4 / wn);
+        // waves along N only as far as N fills them; few tokens (a decode step): all of them along N and tiles of sixteen
+        // tokens, so that the chip has workgroups enough
+        const bool few = n_tokens <= 128;
+        const int wn = few || N > 128 ? 4 : N > 64 ? 2 : 1;
+        const int wg_tokens = few ? 16 : 32 * (4 / wn);
         const int token_tiles = (n_tokens + wg_tokens - 1) / wg_tokens;
         FSIE_REQUIRE(token_tiles <= 65535, "head_gemm: %d tokens are more than one launch takes", n_tokens);
         const dim3 mgrid((N + 64 * wn - 1) / (64 * wn) + turned, token_tiles, heads);
@@ -400,7 +402,7 @@ extern "C" int fsie_head_gemm(const void* x, int64_t x_stride, int x_off, int x_
     head_gemm_mfma_kernel<MT, WN><<<mgrid, kThreads, 0, stream>>>(static_cast<const bf16_t*>(x), x_stride, x_off, x_hs,       \
                                                                 static_cast<const bf16_t*>(w), static_cast<bf16_t*>(y),     \
                                                                 y_stride, y_off, y_hs, ex, n_tokens, heads, N, K, wide)
-        if (n_tokens <= 16) FSIE_HEAD_GEMM(1, 4);
+        if (few) FSIE_HEAD_GEMM(1, 4);
         else if (wn == 4) FSIE_HEAD_GEMM(2, 4);
         else if (wn == 2) FSIE_HEAD_GEMM(2, 2);
         else FSIE_HEAD_GEMM(2, 1);

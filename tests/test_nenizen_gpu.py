@@ -225,7 +225,8 @@ def test_entrance_of_a_pass(ops, dtype, width, rows):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("t, heads, k, n, rot, pairs", [(5, 3, 8, 9, 6, 3), (16, 2, 40, 64, 8, -4), (17, 1, 64, 200, 16, 8), (100, 5, 96, 300, 4, -2),
-                                                        (33, 2, 24, 17, 12, -4), (130, 3, 64, 128, 32, 16), (70, 2, 32, 60, 0, 0), (97, 4, 64, 192, 64, -32)])
+                                                        (33, 2, 24, 17, 12, -4), (130, 3, 64, 128, 32, 16), (70, 2, 32, 60, 0, 0), (97, 4, 64, 192, 64, -32),
+                                                        (129, 2, 40, 60, 8, 4), (161, 2, 64, 192, 16, -8), (300, 2, 72, 100, 10, 5)])
 def test_product_per_head_with_gates_and_turned_parts(ops, dtype, t, heads, k, n, rot, pairs):
     """A factor a head, a gate for every output, both, none; the rotated runs of every head beside the product, zeros
     behind them; the columns in between stay.  Rows that allow 8-byte stores and rows that do not."""
