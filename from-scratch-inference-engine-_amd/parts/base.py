@@ -46,7 +46,7 @@ class ParamDecl:
 
 class HiddenState:
     """The residual stream of a step: ``residual`` float32 [T, H] and a pending ``delta`` that has
-    not been added yet: [T, H] in the compute dtype, or (only if every norm of the model sets
+    not been added yet: [T, H] in the compute dtype (some norms also take it unrounded in float32), or (only if every norm of the model sets
     ``adds_partial_sums``, which the step's context then says in ``partial_sums_ok``) float32
     [S, T, H], partial sums of a matrix product to be added in order.  ``delta_norm``: a norm that the
     pending delta goes through before it is added (a layer that also norms its sublayers' outputs), or
